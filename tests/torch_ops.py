@@ -121,9 +121,10 @@ class TorchOps:
 
     # ---- attention over the paged cache -----------------------------------------------------------------
     def paged_attention(self, q, plane, batch, group, n_heads, n_kv_heads, head_dim, window=0, scale=None, slopes=None,
-                        sink=False, gate=None):
+                        sink=False, gate=None, turn=None):
         n = q.shape[0]
         page_size = plane.shape[3]
+        sinks = self._sinks(sink, n_heads)
         scale = scale if scale is not None else head_dim ** -0.5
         tables = batch.block_tables[group]
         g = n_heads // n_kv_heads
@@ -144,12 +145,29 @@ class TorchOps:
                 s = (k[:, h // g] @ qr[h]) * scale
                 if slopes is not None:
                     s = s + float(slopes[h]) * (js - p).float()
-                w = torch.softmax(torch.cat((s, s.new_zeros(1))), dim=0)[:-1] if sink else torch.softmax(s, dim=0)
+                w = torch.softmax(torch.cat((s, sinks[h:h + 1])), dim=0)[:-1] if sinks is not None else torch.softmax(s, dim=0)
                 o = w @ v[:, h // g]
                 if gate is not None:
                     o = o * torch.sigmoid(gate[r, h].float())
                 out[r, h * head_dim:(h + 1) * head_dim] = o
-        return out.to(q.dtype)
+        return self._turned_back(out, turn, n_heads).to(q.dtype)
+
+    @staticmethod
+    def _sinks(sink, n_heads):
+        """The sink's score per head: False or None for no sink, True for zeros."""
+        if torch.is_tensor(sink):
+            return sink.float()
+        return torch.zeros(n_heads) if sink else None
+
+    @staticmethod
+    def _turned_back(out, turn, n_heads):
+        """Every head's pairs of channels (2m, 2m + 1) turned back by the angles whose (cos, sin) are turn [rows, pairs, 2]."""
+        if turn is None:
+            return out
+        x = out.view(out.shape[0], n_heads, -1)
+        c, s = turn[:, None, :, 0], turn[:, None, :, 1]
+        a, b = x[..., 0::2], x[..., 1::2]
+        return torch.stack((a * c + b * s, b * c - a * s), dim=-1).reshape(out.shape)
 
     def head_gate(self, x, gate, n_heads, vdim):
         y = x.float().view(x.shape[0], n_heads, vdim) * torch.sigmoid(gate.float())[:, :, None]
@@ -239,17 +257,23 @@ class TorchOps:
         return q.reshape(n, H * kd).to(self.dtype)
 
     def latent_prepare(self, proj, q_off, c_off, positions, write_slots, plane, n_heads, dim, rot_dim, rank, page_size,
-                       gain, freqs, rot_dims, eps, write_cache=True):
+                       gain, freqs, rot_dims, eps, write_cache=True, latent=None, pair_half=False, rot_factor=1.0):
         n, H, D, R, C = proj.shape[0], n_heads, dim, rot_dim, rank
+        latent = proj if latent is None else latent
 
         def turned(x):                    # [n, ..., R]
             if not rot_dims:
                 return x
             ang = positions.float()[:, None] * freqs[None, :]
             shape = (n,) + (1,) * (x.dim() - 2) + (rot_dims // 2,)
-            c, s = torch.cos(ang).view(shape), torch.sin(ang).view(shape)
-            a, b = x[..., 0:rot_dims:2], x[..., 1:rot_dims:2]
+            c, s = torch.cos(ang).view(shape) * rot_factor, torch.sin(ang).view(shape) * rot_factor
             y = x.clone()
+            if pair_half:
+                half = rot_dims // 2
+                a, b = x[..., :half], x[..., half:rot_dims]
+                y[..., :half], y[..., half:rot_dims] = a * c - b * s, b * c + a * s
+                return y
+            a, b = x[..., 0:rot_dims:2], x[..., 1:rot_dims:2]
             y[..., 0:rot_dims:2] = a * c - b * s
             y[..., 1:rot_dims:2] = b * c + a * s
             return y
@@ -261,9 +285,9 @@ class TorchOps:
         if D == 0:
             q_plain = torch.zeros(n, H, dtype=self.dtype, device=proj.device)
         if write_cache:
-            c = proj[:, c_off:c_off + C].float()
+            c = latent[:, c_off:c_off + C].float()
             c = c / torch.sqrt((c * c).mean(-1, keepdim=True) + eps) * gain
-            key = torch.cat((c, turned(proj[:, c_off + C:c_off + C + R].float())), dim=-1).to(plane.dtype)
+            key = torch.cat((c, turned(latent[:, c_off + C:c_off + C + R].float())), dim=-1).to(plane.dtype)
             pages = plane.view(plane.shape[0], -1)
             page, off = write_slots.long() // page_size, write_slots.long() % page_size
             pages[:, :page_size * (C + R)].view(-1, page_size, C + R)[page, off] = key
@@ -271,8 +295,9 @@ class TorchOps:
         return q.view(n, H * (C + R)), q_plain
 
     def paged_attention_kv(self, q, plane, batch, group, n_heads, n_kv_heads, key_dim, value_dim, page_size, window=0,
-                           scale=None, sink=False, gate=None, chunk=0):
+                           scale=None, sink=False, gate=None, chunk=0, turn=None):
         n = q.shape[0]
+        sinks = self._sinks(sink, n_heads)
         H, G, kd, vd = n_heads, n_kv_heads, key_dim, value_dim
         scale = scale if scale is not None else kd ** -0.5
         tables = batch.block_tables[group]
@@ -293,18 +318,91 @@ class TorchOps:
             qr = q[r].float().view(H, kd)
             for h in range(H):
                 sc = (k[:, h // (H // G)] @ qr[h]) * scale
-                if sink:
-                    w = torch.softmax(torch.cat((sc, sc.new_zeros(1))), dim=0)[:-1]
+                if sinks is not None:
+                    w = torch.softmax(torch.cat((sc, sinks[h:h + 1])), dim=0)[:-1]
                 else:
                     w = torch.softmax(sc, dim=0)
                 o = w @ v[:, h // (H // G)]
                 if gate is not None:
                     o = o * torch.sigmoid(gate[r, h].float())
                 out[r, h * vd:(h + 1) * vd] = o
-        return out.to(q.dtype)
+        return self._turned_back(out, turn, H).to(q.dtype)
 
-    def latent_attention(self, q, plane, batch, group, n_heads, key_dim, value_dim, page_size, scale):
-        return self.paged_attention_kv(q, plane, batch, group, n_heads, 1, key_dim, value_dim, page_size, 0, scale)
+    def latent_attention(self, q, plane, batch, group, n_heads, key_dim, value_dim, page_size, scale, window=0, sink=None):
+        return self.paged_attention_kv(q, plane, batch, group, n_heads, 1, key_dim, value_dim, page_size, window, scale,
+                                       sink=sink)
+
+    # ---- attention behind a short convolution, with values turned by position -----------------------------------
+    def convolved_prepare(self, proj, bias, taps, state, batch, write_slots, plane, n_heads, n_kv_heads, key_dim, value_dim,
+                          page_size, freqs, rot_dims, rot_factor, turn_freqs, write_cache=True):
+        n = proj.shape[0]
+        H, G, kd, vd = n_heads, n_kv_heads, key_dim, value_dim
+        C, K = taps.shape
+        u = proj[:, :C].float() + bias
+        y = torch.zeros(n, C)
+        cu, slots = batch.cu_rows.tolist(), batch.seq_slots.tolist()
+        for k in range(batch.n_seqs):
+            first, rows = cu[k], cu[k + 1] - cu[k]
+            if rows == 0:
+                continue
+            line = state[slots[k]].view(K - 1, C) if K > 1 else torch.zeros(0, C)
+            seq = torch.cat((line, u[first:first + rows]), dim=0)
+            for j in range(K):
+                y[first:first + rows] += seq[j:j + rows] * taps[:, j]
+            if K > 1:
+                line.copy_(seq[-(K - 1):])
+
+        def turned(x, dims, f, factor):
+            if not dims:
+                return x
+            ang = batch.positions.float()[:, None] * f[None, :]
+            c, s = torch.cos(ang)[:, None, :] * factor, torch.sin(ang)[:, None, :] * factor
+            a, b = x[..., 0:dims:2], x[..., 1:dims:2]
+            out = x.clone()
+            out[..., 0:dims:2], out[..., 1:dims:2] = a * c - b * s, b * c + a * s
+            return out
+
+        q = turned(y[:, :H * kd].view(n, H, kd), rot_dims, freqs, rot_factor)
+        turn = None
+        if turn_freqs is not None:
+            ang = batch.positions.float()[:, None] * turn_freqs[None, :]
+            turn = torch.stack((torch.cos(ang), torch.sin(ang)), dim=-1)
+        if write_cache:
+            k = turned(y[:, H * kd:(H + G) * kd].reshape(n, G, kd), rot_dims, freqs, rot_factor)
+            v = turned(y[:, (H + G) * kd:].reshape(n, G, vd), vd if turn_freqs is not None else 0, turn_freqs, 1.0)
+            pages = plane.view(plane.shape[0], -1)
+            page, off = write_slots.long() // page_size, write_slots.long() % page_size
+            pages[:, :G * page_size * kd].view(-1, G, page_size, kd)[page, :, off] = k.to(plane.dtype)
+            pages[:, G * page_size * kd:].view(-1, G, vd, page_size)[page, :, :, off] = v.to(plane.dtype)
+        return q.reshape(n, H * kd).to(self.dtype), turn
+
+    # ---- a residual of several streams --------------------------------------------------------------------------
+    def mix_streams(self, x, streams, write=None, read=None, shift=None):
+        n, D = x.shape[0], x.shape[-1]
+        if write is not None:
+            y, bias, mix, out = write
+            y = y.float()[:, :D] + (bias if bias is not None else 0.0)
+            X = x if x.dim() == 3 else x[:, None, :].expand(n, streams, D)
+            x = torch.einsum("st,nsd->ntd", mix, X) + out.view(1, streams, 1) * y[:, None, :]
+        if read is None:
+            return x, None
+        weights, gain, eps = read
+        X = x if x.dim() == 3 else x[:, None, :].expand(n, streams, D)
+        u = torch.einsum("s,nsd->nd", weights, X)
+        h = u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * gain
+        if shift is not None:
+            amount, state, batch = shift
+            cu, slots = batch.cu_rows.tolist(), batch.seq_slots.tolist()
+            moved = h.clone()
+            for k in range(batch.n_seqs):
+                first, end = cu[k], cu[k + 1]
+                if end == first:
+                    continue
+                before = torch.cat((state[slots[k]][None, :D], h[first:end - 1]))
+                moved[first:end] = h[first:end] + (before - h[first:end]) * amount
+                state[slots[k], :D] = h[end - 1]
+            h = moved
+        return x, h.to(self.dtype)
 
     # ---- a residual stream in 32-bit, norm before the sublayer ------------------------------------------------
     def layernorm32(self, x32, gain, bias, eps):
@@ -346,9 +444,11 @@ class TorchOps:
         return z
 
     # ---- products in groups ----------------------------------------------------------------------------------
-    def heads_linear(self, x, w, out, out_group, out_offset=0):
+    def heads_linear(self, x, w, out, out_group, out_offset=0, gate=None):
         H, N, K = w.shape
         y = torch.einsum("rhk,hnk->rhn", x.float().view(x.shape[0], H, K), w.float())
+        if gate is not None:
+            y = y * torch.sigmoid(gate.float().reshape(x.shape[0], H, N))
         for h in range(H):
             out[:, out_offset + h * out_group:out_offset + h * out_group + N] = y[:, h].to(out.dtype)
         return out

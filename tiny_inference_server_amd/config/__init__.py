@@ -5,3 +5,4 @@ from .fikevik_config import FikevikConfig
 from .fipuzen_config import FipuzenConfig
 from .rurorax_config import RuroraxConfig
 from .fesupel_config import FesupelConfig
+from .gosavik_config import GosavikConfig

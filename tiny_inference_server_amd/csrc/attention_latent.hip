@@ -12,7 +12,10 @@
 // exactly those eight as its share of P^T, and takes the values of the same eight keys: the contraction's order is
 // free as long as both operands agree. Softmax in 32-bit with a running maximum per column. Slots behind a row's
 // position are read (their page is mapped) but their scores become -inf and their values zero before any arithmetic.
-// A long key range is cut into `n_splits` parts (grid z) whose partial results a second kernel merges.
+// A long key range is cut into `n_splits` parts (grid z) whose partial results a second kernel merges. window > 0: a row
+// sees its last `window` keys only; steps that no row of an item sees are left out, and slots before the first key any
+// row sees (their page may have gone to another request) are treated like those behind the last. sinks (nullable): head h's
+// softmax has one more key of score sinks[h], not scaled, without a value.
 #include "common.h"
 
 TIS_DEFINE_LAST_ERROR(tis_attention_latent)
@@ -34,6 +37,10 @@ __device__ __forceinline__ float quad_max(float v) {      // over the four lanes
   v = fmaxf(v, __shfl_xor(v, 16, 64));
   return fmaxf(v, __shfl_xor(v, 32, 64));
 }
+// what a sink of score `sinks[head]` adds to a denominator whose exponentials are 2^(score * log2(e) - m)
+__device__ __forceinline__ float sink_share(const float* sinks, int head, float m) {
+  return sinks ? exp2f(sinks[head] * 1.4426950408889634f - m) : 0.f;
+}
 __device__ __forceinline__ float quad_sum(float v) {
   v += __shfl_xor(v, 16, 64);
   return v + __shfl_xor(v, 32, 64);
@@ -43,7 +50,7 @@ __global__ __launch_bounds__(64) void latent_mfma_kernel(
     const bf16* __restrict__ q, long ldq, const bf16* __restrict__ plane, const int* __restrict__ block_tables, int bt_ld,
     const int* __restrict__ row_seq, const int* __restrict__ positions, const int2* __restrict__ items,
     bf16* __restrict__ out, long ldo, float* __restrict__ part_o, float2* __restrict__ part_ml, int H, float scale_log2,
-    int n_splits) {
+    int n_splits, int window, const float* __restrict__ sinks) {
   const int item = blockIdx.x, hb = blockIdx.y, split = blockIdx.z;
   const int lane = threadIdx.x, c16 = lane & 15, g = lane >> 4;
   const int row0 = items ? items[item].x : item;
@@ -57,6 +64,8 @@ __global__ __launch_bounds__(64) void latent_mfma_kernel(
   const bool col_ok = ro < n_rows && head < H;
   const int col_row = row0 + (col_ok ? ro : 0);
   const int col_pos = col_ok ? p_first + ro : -1;
+  const int col_lo = window > 0 ? col_pos - window + 1 : 0;                // the column's first key
+  const int k_lo = window > 0 ? max(0, p_first - window + 1) : 0;          // the first key any column sees
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
 
   bf16x8 qb[DC];
@@ -66,9 +75,9 @@ __global__ __launch_bounds__(64) void latent_mfma_kernel(
     qb[dc] = (col_ok && d < KD) ? *reinterpret_cast<const bf16x8*>(q + (long)col_row * ldq + (long)head * KD + d) : zero8;
   }
 
-  const int n_steps = p_last / 32 + 1;
+  const int s_first = k_lo / 32, n_steps = p_last / 32 + 1 - s_first;
   const int per = (n_steps + n_splits - 1) / n_splits;
-  const int s_begin = split * per, s_end = min(n_steps, s_begin + per);
+  const int s_begin = s_first + split * per, s_end = min(s_first + n_steps, s_begin + per);
   f32x4 o[DB];
 #pragma unroll
   for (int db = 0; db < DB; ++db) o[db] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -95,8 +104,8 @@ __global__ __launch_bounds__(64) void latent_mfma_kernel(
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int key0 = kb + 4 * g + i, key1 = key0 + 16;
-      sv[i] = key0 <= col_pos ? st0[i] * scale_log2 : -INFINITY;
-      sv[4 + i] = (ok1 && key1 <= col_pos) ? st1[i] * scale_log2 : -INFINITY;
+      sv[i] = (key0 <= col_pos && key0 >= col_lo) ? st0[i] * scale_log2 : -INFINITY;
+      sv[4 + i] = (ok1 && key1 <= col_pos && key1 >= col_lo) ? st1[i] * scale_log2 : -INFINITY;
       tmax = fmaxf(tmax, fmaxf(sv[i], sv[4 + i]));
     }
     tmax = quad_max(tmax);
@@ -113,18 +122,19 @@ __global__ __launch_bounds__(64) void latent_mfma_kernel(
     }
     l = l * alpha + psum;
     m = m_new;
-    const bool last = kb + 31 > p_last;                        // some of the step's slots lie behind every row
+    const bool edge = kb + 31 > p_last || kb < k_lo;           // some of the step's slots lie behind or before what any row sees
 #pragma unroll
     for (int db = 0; db < DB; ++db) {
       const long off = (long)PAGE * KD + (long)(db * 16 + c16) * PAGE + 4 * g;
       const bf16x4 lo = *reinterpret_cast<const bf16x4*>(pg0 + off);
       const bf16x4 hi = ok1 ? *reinterpret_cast<const bf16x4*>(pg1 + off) : (bf16x4){0, 0, 0, 0};
       bf16x8 va = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
-      if (last) {
+      if (edge) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          if (kb + 4 * g + i > p_last) va[i] = static_cast<__bf16>(0.f);
-          if (kb + 16 + 4 * g + i > p_last) va[4 + i] = static_cast<__bf16>(0.f);
+          const int key0 = kb + 4 * g + i, key1 = key0 + 16;
+          if (key0 > p_last || key0 < k_lo) va[i] = static_cast<__bf16>(0.f);
+          if (key1 > p_last || key1 < k_lo) va[4 + i] = static_cast<__bf16>(0.f);
         }
       }
 #pragma unroll
@@ -137,7 +147,7 @@ __global__ __launch_bounds__(64) void latent_mfma_kernel(
   const float lt = quad_sum(l);
   if (!col_ok) return;
   if (n_splits == 1) {
-    const float inv = 1.f / lt;
+    const float inv = 1.f / (lt + sink_share(sinks, head, m));
     bf16* dst = out + (long)col_row * ldo + (long)head * VD + 4 * g;
 #pragma unroll
     for (int db = 0; db < DB; ++db) {
@@ -166,7 +176,7 @@ static constexpr int TK_BYTES = 32 * TK_STRIDE * 2, TV_BYTES = 2 * VD * PAGE * 2
 __global__ __launch_bounds__(256) void latent_tile_kernel(
     const bf16* __restrict__ q, long ldq, const bf16* __restrict__ plane, const int* __restrict__ block_tables, int bt_ld,
     const int* __restrict__ row_seq, const int* __restrict__ positions, const int2* __restrict__ items,
-    bf16* __restrict__ out, long ldo, int H, float scale_log2) {
+    bf16* __restrict__ out, long ldo, int H, float scale_log2, int window, const float* __restrict__ sinks) {
   __shared__ __attribute__((aligned(16))) bf16 k_lds[32 * TK_STRIDE];
   __shared__ __attribute__((aligned(16))) bf16 v_lds[2 * VD * PAGE];
   const int item = blockIdx.x, hb = blockIdx.y;
@@ -181,6 +191,8 @@ __global__ __launch_bounds__(256) void latent_tile_kernel(
   const bool col_ok = ro < n_rows && head < H && (H >= 64 || c < (64 / H) * H);
   const int col_row = row0 + (col_ok ? ro : 0);
   const int col_pos = col_ok ? p_first + ro : -1;
+  const int col_lo = window > 0 ? col_pos - window + 1 : 0;                // the column's first key
+  const int k_lo = window > 0 ? max(0, p_first - window + 1) : 0;          // the first key any column sees
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
 
   bf16x8 qb[DC];
@@ -194,7 +206,7 @@ __global__ __launch_bounds__(256) void latent_tile_kernel(
   for (int db = 0; db < DB; ++db) o[db] = (f32x4){0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
   const long page_stride = (long)PAGE * (KD + VD);
-  const int n_steps = p_last / 32 + 1;
+  const int s_first = k_lo / 32, n_steps = p_last / 32 + 1;     // (steps s_first .. n_steps - 1)
   constexpr int KP = KD / 8;                                    // 16-byte pieces of a key
   constexpr int VP = VD * PAGE / 8;                             // ... of a page's values
 
@@ -218,8 +230,8 @@ __global__ __launch_bounds__(256) void latent_tile_kernel(
       if (i < 2 * VP) vreg[j] = *reinterpret_cast<const bf16x8*>((pgi ? pg1 : pg0) + (long)PAGE * KD + piece * 8);
     }
   };
-  fetch(0);
-  for (int s = 0; s < n_steps; ++s) {
+  fetch(s_first);
+  for (int s = s_first; s < n_steps; ++s) {
     const int kb = s * 32;
     const bool ok1 = kb + 16 <= p_last;
     __syncthreads();                                            // everyone has read the step before
@@ -249,8 +261,8 @@ __global__ __launch_bounds__(256) void latent_tile_kernel(
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int key0 = kb + 4 * g + i, key1 = key0 + 16;
-      sv[i] = key0 <= col_pos ? st0[i] * scale_log2 : -INFINITY;
-      sv[4 + i] = (ok1 && key1 <= col_pos) ? st1[i] * scale_log2 : -INFINITY;
+      sv[i] = (key0 <= col_pos && key0 >= col_lo) ? st0[i] * scale_log2 : -INFINITY;
+      sv[4 + i] = (ok1 && key1 <= col_pos && key1 >= col_lo) ? st1[i] * scale_log2 : -INFINITY;
       tmax = fmaxf(tmax, fmaxf(sv[i], sv[4 + i]));
     }
     tmax = quad_max(tmax);
@@ -267,18 +279,19 @@ __global__ __launch_bounds__(256) void latent_tile_kernel(
     }
     l = l * alpha + psum;
     m = m_new;
-    const bool last = kb + 31 > p_last;
+    const bool edge = kb + 31 > p_last || kb < k_lo;
 #pragma unroll
     for (int db = 0; db < DB; ++db) {
       const int off = (db * 16 + c16) * PAGE + 4 * g;
       const bf16x4 lo = *reinterpret_cast<const bf16x4*>(v_lds + off);
       const bf16x4 hi = ok1 ? *reinterpret_cast<const bf16x4*>(v_lds + VD * PAGE + off) : (bf16x4){0, 0, 0, 0};
       bf16x8 va = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
-      if (last) {
+      if (edge) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          if (kb + 4 * g + i > p_last) va[i] = static_cast<__bf16>(0.f);
-          if (kb + 16 + 4 * g + i > p_last) va[4 + i] = static_cast<__bf16>(0.f);
+          const int key0 = kb + 4 * g + i, key1 = key0 + 16;
+          if (key0 > p_last || key0 < k_lo) va[i] = static_cast<__bf16>(0.f);
+          if (key1 > p_last || key1 < k_lo) va[4 + i] = static_cast<__bf16>(0.f);
         }
       }
 #pragma unroll
@@ -288,7 +301,7 @@ __global__ __launch_bounds__(256) void latent_tile_kernel(
   }
   const float lt = quad_sum(l);
   if (!col_ok) return;
-  const float inv = 1.f / lt;
+  const float inv = 1.f / (lt + sink_share(sinks, head, m));
   bf16* dst = out + (long)col_row * ldo + (long)head * VD + 4 * g;
 #pragma unroll
   for (int db = 0; db < DB; ++db) {
@@ -301,7 +314,8 @@ __global__ __launch_bounds__(256) void latent_tile_kernel(
 
 // out[row, head, :] = sum_s 2^(m_s - M) o_s / sum_s 2^(m_s - M) l_s over a (row, head)'s splits, in a fixed order
 __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restrict__ part_o, const float2* __restrict__ part_ml,
-                                                           bf16* __restrict__ out, long ldo, int H, int n_splits) {
+                                                           bf16* __restrict__ out, long ldo, int H, int n_splits,
+                                                           const float* __restrict__ sinks) {
   __shared__ float w[256];                 // the weights of up to 256 splits at a time
   __shared__ float red[16];
   const long row = blockIdx.x;
@@ -339,6 +353,7 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restri
       acc[j] += a;
     }
   }
+  L += sink_share(sinks, head, M);         // the sink's share of the denominator, once for all splits
 #pragma unroll
   for (int j = 0; j < (VD + 255) / 256; ++j) {
     const int c = j * 256 + t;
@@ -355,11 +370,11 @@ TIS_EXPORT int tis_attention_latent_dims() { return TIS_LATENT; }
 TIS_EXPORT int tis_attention_latent(const void* q, long ldq, const void* plane, const int* block_tables, int bt_ld,
                                     const int* row_seq, const int* positions, const int* items, int n_items, void* out,
                                     long ldo, float* part_o, float* part_ml, int rows, int H, int key_dim, int value_dim,
-                                    int page_size, float scale, int n_splits, hipStream_t stream) {
+                                    int page_size, float scale, int n_splits, int window, const float* sinks, hipStream_t stream) {
   if (rows == 0 || n_items == 0) return 0;
   if (key_dim != KD || value_dim != VD) return tis_fail("attention_latent: built for keys of %d and values of %d, called with %d and %d", KD, VD, key_dim, value_dim);
   if (page_size != PAGE) return tis_fail("attention_latent: pages of %d slots (this kernel takes %d)", page_size, PAGE);
-  if (rows < 0 || n_items < 0 || H < 1 || n_splits < 0 || n_splits > 65535 || (H + 15) / 16 > 65535)
+  if (rows < 0 || n_items < 0 || H < 1 || window < 0 || n_splits < 0 || n_splits > 65535 || (H + 15) / 16 > 65535)
     return tis_fail("attention_latent: bad size rows=%d items=%d heads=%d splits=%d", rows, n_items, H, n_splits);
   if (n_splits > 1 && (!part_o || !part_ml)) return tis_fail("attention_latent: %d splits need a workspace", n_splits);
   if ((ldq % 8) || (ldo % 4) || ((uintptr_t)q % 16) || ((uintptr_t)out % 8) || ((uintptr_t)plane % 16))
@@ -369,16 +384,16 @@ TIS_EXPORT int tis_attention_latent(const void* q, long ldq, const void* plane, 
     dim3 tgrid(n_items, (H + 63) / 64);
     latent_tile_kernel<<<tgrid, 256, 0, stream>>>((const bf16*)q, ldq, (const bf16*)plane, block_tables, bt_ld, row_seq,
                                                   positions, (const int2*)items, (bf16*)out, ldo, H,
-                                                  scale * 1.4426950408889634f);
+                                                  scale * 1.4426950408889634f, window, sinks);
     return tis_launch_status("attention_latent tiles");
   }
   dim3 grid(n_items, (H + 15) / 16, n_splits);
   latent_mfma_kernel<<<grid, 64, 0, stream>>>((const bf16*)q, ldq, (const bf16*)plane, block_tables, bt_ld, row_seq, positions,
                                              (const int2*)items, (bf16*)out, ldo, part_o, (float2*)part_ml, H,
-                                             scale * 1.4426950408889634f, n_splits);
+                                             scale * 1.4426950408889634f, n_splits, window, sinks);
   int rc = tis_launch_status("attention_latent");
   if (rc || n_splits == 1) return rc;
   dim3 mgrid(rows, H);
-  latent_merge_kernel<<<mgrid, 256, 0, stream>>>(part_o, (const float2*)part_ml, (bf16*)out, ldo, H, n_splits);
+  latent_merge_kernel<<<mgrid, 256, 0, stream>>>(part_o, (const float2*)part_ml, (bf16*)out, ldo, H, n_splits, sinks);
   return tis_launch_status("attention_latent merge");
 }

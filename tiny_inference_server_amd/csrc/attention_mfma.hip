@@ -78,6 +78,11 @@ __device__ __forceinline__ float column_sum(float v) {
   return __uint_as_float(b[0]) + __uint_as_float(b[1]);
 }
 
+// What a sink adds to a denominator whose exponentials are 2^(score * log2(e) - m): its score is sinks[head], or 0.
+__device__ __forceinline__ float sink_share(const float* sinks, int head, float m) {
+  return __builtin_amdgcn_exp2f((sinks ? sinks[head] * 1.4426950408889634f : 0.f) - m);
+}
+
 // PS16: pages of exactly 16 tokens. A 16-key tile is then a whole page, page indices are shifts, and a lane's
 // offsets inside a page never change: the loads of a step need no address arithmetic beyond the page's base.
 template <int NB, bool PS16>
@@ -86,7 +91,7 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(NB <= 2 ? 2 
     int bt_ld, const int* __restrict__ row_seq, const int* __restrict__ positions, const int2* __restrict__ items,
     bf16* __restrict__ out, long out_ld, float* __restrict__ part_o, float2* __restrict__ part_ml, int group_size,
     int n_kv_heads, int n_heads, int page_size_arg, int window, float scale_log2, int n_splits, int min_steps,
-    int split_stride, int* __restrict__ row_splits, int sink) {
+    int split_stride, int* __restrict__ row_splits, int sink, const float* __restrict__ sinks) {
   const int page_size = PS16 ? 16 : page_size_arg;
   const int item = blockIdx.x, kvh = blockIdx.y;
   int split = blockIdx.z;
@@ -357,7 +362,7 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(NB <= 2 ? 2 
     if (!col_ok[nb]) continue;
     if (item_splits == 1) {
       // a sink: one more key of score 0 without a value, which only the denominator sees
-      const float inv = 1.f / (sink ? lt + __builtin_amdgcn_exp2f(-m[nb]) : lt);
+      const float inv = 1.f / (sink ? lt + sink_share(sinks, col_head[nb], m[nb]) : lt);
       bf16* dst = out + (long)col_row[nb] * out_ld + (long)col_head[nb] * HD + g * 4;
 #pragma unroll
       for (int db = 0; db < DB; ++db) {
@@ -443,7 +448,7 @@ __global__ __launch_bounds__(TW * 64) __attribute__((amdgpu_waves_per_eu(HD <= 1
     int bt_ld, const int* __restrict__ row_seq, const int* __restrict__ positions, const int2* __restrict__ tiles,
     bf16* __restrict__ out, long out_ld, float* __restrict__ part_o, float2* __restrict__ part_ml, int group_size,
     int n_kv_heads, int n_heads, int page_size_arg, int window, float scale_log2, int n_splits, int max_steps,
-    int split_stride, int* __restrict__ row_splits, int sink) {
+    int split_stride, int* __restrict__ row_splits, int sink, const float* __restrict__ sinks) {
   __shared__ __attribute__((aligned(16))) bf16 k_lds[TBUF][TCH * 8];
   __shared__ __attribute__((aligned(16))) bf16 v_lds[TBUF][TCH * 8];
   const int page_size = PS16 ? 16 : page_size_arg;
@@ -717,7 +722,7 @@ __global__ __launch_bounds__(TW * 64) __attribute__((amdgpu_waves_per_eu(HD <= 1
   const float lt = pair_sum(l);
   if (!col_ok) return;
   if (item_splits == 1) {
-    const float inv = 1.f / (sink ? lt + __builtin_amdgcn_exp2f(-m) : lt);
+    const float inv = 1.f / (sink ? lt + sink_share(sinks, col_head, m) : lt);
     bf16* dst = out + (long)col_row * out_ld + (long)col_head * HD + h * 4;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt)
@@ -753,7 +758,7 @@ __global__ __launch_bounds__(MG * 64) void attention_merge_kernel(const float* _
                                                                   const float2* __restrict__ part_ml,
                                                                   bf16* __restrict__ out, long out_ld, int n_heads,
                                                                   int max_splits, const int* __restrict__ row_splits,
-                                                                  int sink) {
+                                                                  int sink, const float* __restrict__ sinks) {
   __shared__ float so[MG][MD][64];
   const long row = blockIdx.x;
   const int head = blockIdx.y;
@@ -803,7 +808,7 @@ __global__ __launch_bounds__(MG * 64) void attention_merge_kernel(const float* _
   }
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) L += __shfl_xor(L, off, 64);
-  if (sink) L += exp2f(-M);      // the sink's share of the denominator, once for all splits
+  if (sink) L += sink_share(sinks, head, M);      // the sink's share of the denominator, once for all splits
 #pragma unroll
   for (int j = 0; j < MD; ++j) so[grp][j][lane] = acc[j];
   __syncthreads();
@@ -827,7 +832,7 @@ __global__ __launch_bounds__(MG * 64) void attention_merge_rows_kernel(const flo
                                                                        const float2* __restrict__ part_ml,
                                                                        bf16* __restrict__ out, long out_ld,
                                                                        int n_heads, int max_splits,
-                                                                       const int* __restrict__ row_splits, int sink) {
+                                                                       const int* __restrict__ row_splits, int sink, const float* __restrict__ sinks) {
   const long row = blockIdx.x;
   const int n_splits = row_splits ? row_splits[row] : max_splits;
   if (n_splits <= 1) return;
@@ -864,7 +869,7 @@ __global__ __launch_bounds__(MG * 64) void attention_merge_rows_kernel(const flo
   }
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) L += __shfl_xor(L, off, 64);
-  if (sink) L += exp2f(-M);
+  if (sink) L += sink_share(sinks, head, M);
 #pragma unroll
   for (int j = 0; j < MD; ++j) {
     const int d = j * 64 + lane;
@@ -929,7 +934,7 @@ static int attention_launch(const void* q, long q_ld, const void* plane, const i
                             const int* tiles, int n_tiles, void* out, long out_ld, float* part_o,
                             float* part_ml, int rows, int n_heads, int n_kv_heads, int head_dim, int page_size,
                             int window, float scale, int n_splits, int min_steps, int tile_splits,
-                            int tile_max_steps, int* row_splits, hipStream_t stream, int sink = 0) {
+                            int tile_max_steps, int* row_splits, hipStream_t stream, int sink = 0, const float* sinks = nullptr) {
   if ((n_items == 0 && n_tiles == 0) || rows == 0) return 0;
   if (n_items < 0 || n_tiles < 0 || (n_tiles > 0 && !tiles)) return tis_fail("attention_mfma: bad item counts %d, %d", n_items, n_tiles);
   if (head_dim != HD) return tis_fail("attention_mfma: built for head size %d, called with %d", HD, head_dim);
@@ -989,7 +994,7 @@ static int attention_launch(const void* q, long q_ld, const void* plane, const i
   attention_mfma_kernel<NBV, PSV><<<grid, 64, 0, stream>>>(                                                      \
       (const bf16*)q, q_ld, (const bf16*)plane, block_tables, bt_ld, row_seq, positions, (const int2*)items,     \
       (bf16*)out, out_ld, part_o, (float2*)part_ml, group, n_kv_heads, n_heads, page_size, window, scale_log2,   \
-      n_splits, min_steps, stride, row_splits, sink)
+      n_splits, min_steps, stride, row_splits, sink, sinks)
     if (page_size == 16) {
       if (nb == 1) LAUNCH(1, true);
       else if (nb == 2) LAUNCH(2, true);
@@ -1008,7 +1013,7 @@ static int attention_launch(const void* q, long q_ld, const void* plane, const i
   attention_tile_kernel<PSV><<<grid, TW * 64, 0, tile_stream>>>(                                                      \
       (const bf16*)q, q_ld, (const bf16*)plane, block_tables, bt_ld, row_seq, positions, (const int2*)tiles,     \
       (bf16*)out, out_ld, part_o, (float2*)part_ml, group, n_kv_heads, n_heads, page_size, window, scale_log2,   \
-      tile_splits, tile_max_steps, stride, row_splits, sink)
+      tile_splits, tile_max_steps, stride, row_splits, sink, sinks)
     if (page_size == 16) LAUNCH(true);
     else LAUNCH(false);
 #undef LAUNCH
@@ -1022,11 +1027,11 @@ static int attention_launch(const void* q, long q_ld, const void* plane, const i
     if ((long)rows * n_heads > 8192) {
       dim3 mgrid(rows, (n_heads + MG - 1) / MG);
       attention_merge_rows_kernel<<<mgrid, MG * 64, 0, stream>>>(part_o, (const float2*)part_ml, (bf16*)out, out_ld,
-                                                                 n_heads, stride, row_splits, sink);
+                                                                 n_heads, stride, row_splits, sink, sinks);
     } else {
       dim3 mgrid(rows, n_heads);
       attention_merge_kernel<<<mgrid, MG * 64, 0, stream>>>(part_o, (const float2*)part_ml, (bf16*)out, out_ld,
-                                                            n_heads, stride, row_splits, sink);
+                                                            n_heads, stride, row_splits, sink, sinks);
     }
     rc = tis_launch_status("attention_merge");
   }
@@ -1044,17 +1049,18 @@ TIS_EXPORT int tis_attention_mfma(const void* q, long q_ld, const void* plane, c
                           n_splits, min_steps, tile_splits, tile_max_steps, row_splits, stream);
 }
 
-// The same with a sink in every row's softmax (sink != 0): the denominator also counts one key of score 0 that has no
-// value, so a row's weights add up to less than one.
+// The same with a sink in every row's softmax (sink != 0): the denominator also counts one key that has no value, of score
+// 0 or (sinks not null, one number per query head) sinks[head], which is not scaled; a row's weights add up to less than one.
 TIS_EXPORT int tis_attention_mfma_sink(const void* q, long q_ld, const void* plane, const int* block_tables, int bt_ld,
                                        const int* row_seq, const int* positions, const int* items, int n_items, int nb,
                                        const int* tiles, int n_tiles, void* out, long out_ld, float* part_o,
                                        float* part_ml, int rows, int n_heads, int n_kv_heads, int head_dim, int page_size,
                                        int window, float scale, int n_splits, int min_steps, int tile_splits,
-                                       int tile_max_steps, int* row_splits, int sink, hipStream_t stream) {
+                                       int tile_max_steps, int* row_splits, int sink, const float* sinks,
+                                       hipStream_t stream) {
   return attention_launch(q, q_ld, plane, block_tables, bt_ld, row_seq, positions, items, n_items, nb, tiles, n_tiles,
                           out, out_ld, part_o, part_ml, rows, n_heads, n_kv_heads, head_dim, page_size, window, scale,
-                          n_splits, min_steps, tile_splits, tile_max_steps, row_splits, stream, sink);
+                          n_splits, min_steps, tile_splits, tile_max_steps, row_splits, stream, sink, sinks);
 }
 
 // ---- the same without a workspace argument: partial results in memory that this library owns for good ----

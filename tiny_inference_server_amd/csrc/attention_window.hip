@@ -176,19 +176,20 @@ __global__ __launch_bounds__(1024) void attention_prepare_row_kernel(
 }
 
 // The same step where all heads share one latent as keys and values. grid (rows, H + 1), one wave each.
-// (A latent's pages are those of one key/value head with keys of C + R and values of C channels: the latent is kept
+// (The queries' projections and the latent's may be two matrices. A latent's pages are those of one key/value head with keys of C + R and values of C channels: the latent is kept
 // twice, as the first channels of its key and transposed as its value.) Unit u < H, a query head: the head's R rotated channels (32-bit, at q_off + u * (D + R) + D of proj) are turned by
 // the row's position and written to q_out[u * (C + R) + C ...]; its D unrotated channels go, in the compute type, to
 // q_plain[u * D ...] (for the product that takes them into the latent's space, whose result belongs to
 // q_out[u * (C + R) ...]). Unit H: the row's latent, C channels at c_off, RMS-normed with `gain`, then the R channels
 // of the shared rotated key, turned alike; both go into the row's slot of the page's keys, and the latent also into
-// its values.
+// its values. pair_half: the rotated pairs are (i, i + rot_dims / 2) instead of (2i, 2i + 1); rot_factor multiplies cosine
+// and sine.
 template <typename T>
 __global__ __launch_bounds__(TIS_WAVE) void latent_prepare_kernel(
-    const float* __restrict__ proj, long ldp, int q_off, int c_off, const int* __restrict__ positions,
-    const int* __restrict__ write_slots, T* __restrict__ plane, T* __restrict__ q_out, long ldq, T* __restrict__ q_plain,
-    long ldqp, const float* __restrict__ gain, const float* __restrict__ freqs, int rot_dims, float eps, int H, int D,
-    int R, int C, int page_size) {
+    const float* __restrict__ proj, long ldp, int q_off, const float* __restrict__ latent, long ldl, int c_off,
+    const int* __restrict__ positions, const int* __restrict__ write_slots, T* __restrict__ plane, T* __restrict__ q_out,
+    long ldq, T* __restrict__ q_plain, long ldqp, const float* __restrict__ gain, const float* __restrict__ freqs, int rot_dims,
+    int pair_half, float rot_factor, float eps, int H, int D, int R, int C, int page_size) {
   const long r = blockIdx.x;
   const int u = blockIdx.y, lane = threadIdx.x;
   const float pos = (float)positions[r];
@@ -205,7 +206,7 @@ __global__ __launch_bounds__(TIS_WAVE) void latent_prepare_kernel(
     T* page = plane + (long)(ws / page_size) * page_size * (2 * C + R);
     T* key = page + (long)(ws % page_size) * (C + R);
     T* val = page + (long)page_size * (C + R) + ws % page_size;
-    src = proj + r * ldp + c_off;
+    src = latent + r * ldl + c_off;
     float ss = 0.f;
     for (int e = lane; e < C; e += TIS_WAVE) ss += src[e] * src[e];
     ss = wave_sum(ss);
@@ -218,12 +219,16 @@ __global__ __launch_bounds__(TIS_WAVE) void latent_prepare_kernel(
     src += C;
     dst = key + C;
   }
+  const int half = rot_dims / 2;
   for (int p = lane; 2 * p < R; p += TIS_WAVE) {
-    const int e0 = 2 * p, e1 = e0 + 1;
+    // (with pairs of halves the channels behind the rotated ones are taken two by two)
+    const int e0 = pair_half && p < half ? p : 2 * p, e1 = pair_half && p < half ? p + half : e0 + 1;
     float x = src[e0], y = e1 < R ? src[e1] : 0.f;
-    if (e1 < rot_dims) {
+    if (p < half) {
       float sn, cs;
       sincosf(pos * freqs[p], &sn, &cs);
+      sn *= rot_factor;
+      cs *= rot_factor;
       const float rx = x * cs - y * sn, ry = y * cs + x * sn;
       x = rx;
       y = ry;
@@ -235,13 +240,15 @@ __global__ __launch_bounds__(TIS_WAVE) void latent_prepare_kernel(
 
 // One workgroup per (row, query head). Keys are walked in chunks of AW_CHUNK with a running maximum; the order of
 // every sum depends on the row's own position and window only. sink: the softmax's denominator also holds a key of
-// score 0 that has no value. gate (nullable): the head's result is multiplied by sigmoid(gate[row * ldg + head]).
+// score 0, or of score sinks[head] where that is given, that has no value. gate (nullable): the head's result is multiplied
+// by sigmoid(gate[row * ldg + head]). turn (nullable): the pairs (2m, 2m + 1) of the head's result are turned back by the
+// angle whose (cos, sin) is turn[row * VD / 2 + m].
 template <typename T>
 __global__ __launch_bounds__(AW_THREADS) void attention_window_kernel(
     const T* __restrict__ q, long ldq, const T* __restrict__ plane, const int* __restrict__ block_tables, int bt_ld,
     const int* __restrict__ row_seq, const int* __restrict__ positions, T* __restrict__ out, long ldo, int group_size,
     int G, int KD, int VD, int page_size, int window, int chunk_size, float scale, int sink,
-    const float* __restrict__ gate, long ldg) {
+    const float* __restrict__ sinks, const float* __restrict__ gate, long ldg, const float2* __restrict__ turn) {
   __shared__ float qs[AW_MAX_DIM];
   __shared__ float sc[AW_CHUNK];
   __shared__ float red[16];
@@ -264,7 +271,7 @@ __global__ __launch_bounds__(AW_THREADS) void attention_window_kernel(
   const int lanes_per_key = AW_THREADS / width;
   const int part = t / width, d = t % width;
   const bool pv = part < lanes_per_key;
-  float m = sink ? 0.f : -INFINITY, l = sink ? 1.f : 0.f;
+  float m = sink ? (sinks ? sinks[h] : 0.f) : -INFINITY, l = sink ? 1.f : 0.f;
   float acc[AW_PER];
 #pragma unroll
   for (int u = 0; u < AW_PER; ++u) acc[u] = 0.f;
@@ -309,10 +316,18 @@ __global__ __launch_bounds__(AW_THREADS) void attention_window_kernel(
   for (int u = 0; u < AW_PER; ++u) accm[u][t] = pv ? acc[u] : 0.f;
   __syncthreads();
   const float mul = (gate ? 1.f / (1.f + expf(-gate[r * ldg + h])) : 1.f) / l;
-  for (int c = t; c < VD; c += AW_THREADS) {
+  auto channel = [&](int c) {
     const int u = c / width, dd = c % width;
     float o = 0.f;
     for (int p = 0; p < lanes_per_key; ++p) o += accm[u][p * width + dd];
+    return o;
+  };
+  for (int c = t; c < VD; c += AW_THREADS) {
+    float o = channel(c);
+    if (turn) {
+      const float2 cs = turn[r * (VD / 2) + c / 2];
+      o = c % 2 ? o * cs.x - channel(c - 1) * cs.y : o * cs.x + channel(c + 1) * cs.y;
+    }
     out[r * ldo + (long)h * VD + c] = from_f<T>(o * mul);
   }
 }
@@ -358,10 +373,11 @@ TIS_EXPORT int tis_attention_prepare(int dtype, const float* proj, long ldp, int
   return tis_launch_status("attention_prepare");
 }
 
-TIS_EXPORT int tis_latent_prepare(int dtype, const float* proj, long ldp, int q_off, int c_off, const int* positions,
-                                  const int* write_slots, void* plane, void* q_out, long ldq, void* q_plain, long ldqp,
-                                  const float* gain, const float* freqs, int rot_dims, float eps, int rows, int H, int D,
-                                  int R, int C, int page_size, hipStream_t stream) {
+TIS_EXPORT int tis_latent_prepare(int dtype, const float* proj, long ldp, int q_off, const float* latent, long ldl, int c_off,
+                                  const int* positions, const int* write_slots, void* plane, void* q_out, long ldq,
+                                  void* q_plain, long ldqp, const float* gain, const float* freqs, int rot_dims, int pair_half,
+                                  float rot_factor, float eps, int rows, int H, int D, int R, int C, int page_size,
+                                  hipStream_t stream) {
   if (rows == 0) return 0;
   if (rows < 0 || H < 1 || H > 65534 || D < 0 || R < 0 || C < 1 || page_size < 1 || !gain || !q_out || (D && !q_plain))
     return tis_fail("latent_prepare: bad size rows=%d heads=%d dim=%d rotated=%d latent=%d page=%d", rows, H, D, R, C, page_size);
@@ -370,11 +386,13 @@ TIS_EXPORT int tis_latent_prepare(int dtype, const float* proj, long ldp, int q_
   if (write_slots && !plane) return tis_fail("latent_prepare: write slots without pages");
   dim3 grid(rows, H + 1);
   if (dtype == TIS_F32)
-    latent_prepare_kernel<float><<<grid, TIS_WAVE, 0, stream>>>(proj, ldp, q_off, c_off, positions, write_slots, (float*)plane,
-        (float*)q_out, ldq, (float*)q_plain, ldqp, gain, freqs, rot_dims, eps, H, D, R, C, page_size);
+    latent_prepare_kernel<float><<<grid, TIS_WAVE, 0, stream>>>(proj, ldp, q_off, latent, ldl, c_off, positions, write_slots,
+        (float*)plane, (float*)q_out, ldq, (float*)q_plain, ldqp, gain, freqs, rot_dims, pair_half, rot_factor, eps, H, D, R, C,
+        page_size);
   else if (dtype == TIS_BF16)
-    latent_prepare_kernel<bf16><<<grid, TIS_WAVE, 0, stream>>>(proj, ldp, q_off, c_off, positions, write_slots, (bf16*)plane,
-        (bf16*)q_out, ldq, (bf16*)q_plain, ldqp, gain, freqs, rot_dims, eps, H, D, R, C, page_size);
+    latent_prepare_kernel<bf16><<<grid, TIS_WAVE, 0, stream>>>(proj, ldp, q_off, latent, ldl, c_off, positions, write_slots,
+        (bf16*)plane, (bf16*)q_out, ldq, (bf16*)q_plain, ldqp, gain, freqs, rot_dims, pair_half, rot_factor, eps, H, D, R, C,
+        page_size);
   else
     return tis_fail("unknown dtype code %d", dtype);
   return tis_launch_status("latent_prepare");
@@ -383,19 +401,23 @@ TIS_EXPORT int tis_latent_prepare(int dtype, const float* proj, long ldp, int q_
 TIS_EXPORT int tis_attention_window(int dtype, const void* q, long ldq, const void* plane, const int* block_tables,
                                     int bt_ld, const int* row_seq, const int* positions, void* out, long ldo, int rows,
                                     int H, int G, int KD, int VD, int page_size, int window, int chunk_size, float scale,
-                                    int sink, const float* gate, long ldg, hipStream_t stream) {
+                                    int sink, const float* sinks, const float* gate, long ldg, const float* turn,
+                                    hipStream_t stream) {
   if (rows == 0) return 0;
   if (rows < 0 || H < 1 || G < 1 || H % G || page_size < 1 || window < 0 || chunk_size < 0 || H > 65535)
     return tis_fail("attention_window: bad size rows=%d heads=%d kv_heads=%d page=%d window=%d", rows, H, G, page_size, window);
   if (KD < 1 || KD > AW_MAX_DIM || VD < 1 || VD > AW_MAX_DIM)
     return tis_fail("attention_window: key size %d or value size %d is outside 1..%d", KD, VD, AW_MAX_DIM);
+  if (turn && VD % 2) return tis_fail("attention_window: values of %d channels cannot be turned back in pairs", VD);
   dim3 grid(rows, H);
   if (dtype == TIS_F32)
     attention_window_kernel<float><<<grid, AW_THREADS, 0, stream>>>((const float*)q, ldq, (const float*)plane, block_tables,
-        bt_ld, row_seq, positions, (float*)out, ldo, H / G, G, KD, VD, page_size, window, chunk_size, scale, sink, gate, ldg);
+        bt_ld, row_seq, positions, (float*)out, ldo, H / G, G, KD, VD, page_size, window, chunk_size, scale, sink, sinks, gate,
+        ldg, (const float2*)turn);
   else if (dtype == TIS_BF16)
     attention_window_kernel<bf16><<<grid, AW_THREADS, 0, stream>>>((const bf16*)q, ldq, (const bf16*)plane, block_tables,
-        bt_ld, row_seq, positions, (bf16*)out, ldo, H / G, G, KD, VD, page_size, window, chunk_size, scale, sink, gate, ldg);
+        bt_ld, row_seq, positions, (bf16*)out, ldo, H / G, G, KD, VD, page_size, window, chunk_size, scale, sink, sinks, gate,
+        ldg, (const float2*)turn);
   else
     return tis_fail("unknown dtype code %d", dtype);
   return tis_launch_status("attention_window");

@@ -153,9 +153,18 @@ struct GroupedArgs {
   int line, rows, a_div;
   long lda, a_group, ldc, c_group;
   int N, K, act;        // act 0: none, 1: erf-form gelu
+  const float* gate = nullptr;      // [rows][ldg], N columns a group: a result times sigmoid of its number; null: as it is
+  long ldg = 0;
 };
 
 // plain multiply-adds, any type and any alignment: 16 entries x 64 columns a workgroup, K in steps of 32 through LDS
+// What becomes of entry e's sum for column n of group g.
+__device__ __forceinline__ float grouped_result(const GroupedArgs& p, float v, int e, int g, int n) {
+  if (p.act == 1) v = gelu_erf_f(v);
+  if (p.gate) v *= 1.f / (1.f + expf(-p.gate[(long)e * p.ldg + (long)g * p.N + n]));
+  return v;
+}
+
 template <typename TA, typename TO>
 __global__ __launch_bounds__(256) void grouped_plain_kernel(const TA* __restrict__ A, const TA* __restrict__ W,
                                                             TO* __restrict__ C, GroupedArgs p) {
@@ -193,7 +202,7 @@ __global__ __launch_bounds__(256) void grouped_plain_kernel(const TA* __restrict
   for (int i = 0; i < 4; ++i) {
     const int e = entry[ty * 4 + i];
     if (e < 0) continue;
-    const float v = p.act == 1 ? gelu_erf_f(acc[i]) : acc[i];
+    const float v = grouped_result(p, acc[i], e, g, n0 + tx);
     C[(long)e * p.ldc + (long)g * p.c_group + n0 + tx] = from_f<TO>(v);
   }
 }
@@ -267,7 +276,7 @@ __global__ __launch_bounds__(256) void grouped_mfma_kernel(const bf16* __restric
       for (int e = 0; e < 4; ++e) {
         const int n = n0 + j * 16 + 4 * kg + e;
         if (n >= p.N) continue;
-        const float v = p.act == 1 ? gelu_erf_f(acc[i][j][e]) : acc[i][j][e];
+        const float v = grouped_result(p, acc[i][j][e], mine[i], g, n);
         C[(long)mine[i] * p.ldc + (long)g * p.c_group + n] = from_f<TO>(v);
       }
   }
@@ -376,7 +385,7 @@ __global__ __launch_bounds__(256) void grouped_tiles_kernel(const bf16* __restri
         if (n >= p.N) continue;               // (N is a multiple of 4: the four columns are inside or outside together)
         float v[4];
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = p.act == 1 ? gelu_erf_f(acc[i][j][q * 4 + e]) : acc[i][j][q * 4 + e];
+        for (int e = 0; e < 4; ++e) v[e] = grouped_result(p, acc[i][j][q * 4 + e], entry(m), g, n + e);
         if constexpr (sizeof(TO) == 4) {
           *(f32x4*)(dst + n) = (f32x4){v[0], v[1], v[2], v[3]};
         } else {
@@ -431,14 +440,16 @@ TIS_EXPORT int tis_expert_lists(const int* ids, int n_assign, int n_experts, int
 // group can have (the grid's height).
 TIS_EXPORT int tis_grouped_linear(int in_dtype, int out_dtype, const void* A, long lda, long a_group, int a_div, const void* W,
                                   void* C, long ldc, long c_group, const int* lists, const int* counts, int line,
-                                  int groups, int most_rows, int N, int K, int act, hipStream_t stream) {
+                                  int groups, int most_rows, int N, int K, int act, const float* gate, long ldg,
+                                  hipStream_t stream) {
   if (groups == 0 || most_rows == 0) return 0;
   if (groups < 0 || groups > 65535 || most_rows < 0 || N < 1 || K < 1 || a_div < 1 || (act != 0 && act != 1))
     return tis_fail("grouped_linear: bad size groups=%d rows=%d N=%d K=%d", groups, most_rows, N, K);
+  if (gate && (lists || act)) return tis_fail("grouped_linear: a gate goes with groups of all rows and no activation");
   if ((lists == nullptr) != (counts == nullptr)) return tis_fail("grouped_linear: lists and counts go together");
   const int tiles_m = (most_rows + 15) / 16;
   if (tiles_m > 65535) return tis_fail("grouped_linear: %d rows are too many for one call", most_rows);
-  GroupedArgs p{lists, counts, line, most_rows, a_div, lda, a_group, ldc, c_group, N, K, act};
+  GroupedArgs p{lists, counts, line, most_rows, a_div, lda, a_group, ldc, c_group, N, K, act, gate, ldg};
   dim3 grid((N + 63) / 64, tiles_m, groups);
   if (in_dtype == TIS_BF16) {
     const bool aligned = K % 8 == 0 && lda % 8 == 0 && a_group % 8 == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0;

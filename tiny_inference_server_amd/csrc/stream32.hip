@@ -81,18 +81,18 @@ __global__ __launch_bounds__(S32_THREADS) void gated_postnorm_kernel(
 
 // out = x / sqrt(mean(x^2) + eps) * gain, from the 32-bit stream into the compute type
 template <typename T>
-__global__ __launch_bounds__(S32_THREADS) void rmsnorm32_kernel(const float* __restrict__ x, const float* __restrict__ gain,
+__global__ __launch_bounds__(S32_THREADS) void rmsnorm32_kernel(const float* __restrict__ x, long ldx, const float* __restrict__ gain,
                                                                  float eps, T* __restrict__ out, long ldo, int D) {
   __shared__ float red[16];
   const long r = blockIdx.x;
   float ss = 0.f;
   for (int c = threadIdx.x; c < D; c += S32_THREADS) {
-    const float v = x[r * D + c];
+    const float v = x[r * ldx + c];
     ss += v * v;
   }
   ss = block_sum(ss, red);
   const float inv = 1.f / sqrtf(ss / (float)D + eps);
-  for (int c = threadIdx.x; c < D; c += S32_THREADS) out[r * ldo + c] = from_f<T>(x[r * D + c] * inv * gain[c]);
+  for (int c = threadIdx.x; c < D; c += S32_THREADS) out[r * ldo + c] = from_f<T>(x[r * ldx + c] * inv * gain[c]);
 }
 
 // One wave per (row, head): o / sqrt(mean_over_V(o^2) + eps) * gain * act(g). gain is [V] shared by the heads or
@@ -358,12 +358,12 @@ TIS_EXPORT int tis_gated_postnorm(int dtype, const float* x, const float* y0, lo
   return tis_launch_status("gated_postnorm");
 }
 
-TIS_EXPORT int tis_rmsnorm32(int dtype, const float* x, const float* gain, float eps, void* out, long ldo, int rows, int D,
+TIS_EXPORT int tis_rmsnorm32(int dtype, const float* x, long ldx, const float* gain, float eps, void* out, long ldo, int rows, int D,
                              hipStream_t stream) {
   if (rows == 0) return 0;
   if (rows < 0 || D < 1) return tis_fail("rmsnorm32: bad size rows=%d width=%d", rows, D);
-  S32_DISPATCH((rmsnorm32_kernel<float><<<rows, S32_THREADS, 0, stream>>>(x, gain, eps, (float*)out, ldo, D)),
-               (rmsnorm32_kernel<bf16><<<rows, S32_THREADS, 0, stream>>>(x, gain, eps, (bf16*)out, ldo, D)))
+  S32_DISPATCH((rmsnorm32_kernel<float><<<rows, S32_THREADS, 0, stream>>>(x, ldx, gain, eps, (float*)out, ldo, D)),
+               (rmsnorm32_kernel<bf16><<<rows, S32_THREADS, 0, stream>>>(x, ldx, gain, eps, (bf16*)out, ldo, D)))
   return tis_launch_status("rmsnorm32");
 }
 

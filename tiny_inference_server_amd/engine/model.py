@@ -5,7 +5,7 @@ them, whose cache a call uses, where a stage's rows come from and which norm clo
 """
 from __future__ import annotations
 
-from typing import Dict, List, Optional
+from typing import Dict, List, Optional, Tuple
 
 import torch
 
@@ -50,26 +50,34 @@ class Model:
         self.reads_previous = [bool(getattr(part_class(st.input), "reads_previous", False)) for st in spec.stages]
         if self.reads_previous and self.reads_previous[0]:
             raise ValueError("the first stage cannot read a previous stage")
-        # cache keys: one per call and mixer part unless the call names another's; a block with one mixer uses the
-        # call's key as it is, a block with several appends the part's name
-        self.call_keys: List[List[Dict[str, str]]] = []
+        # cache keys: one per call and part that keeps something unless the call names another's; a block with one such
+        # part uses the call's key as it is, a block with several appends the part's name. A part that keeps both pages and
+        # a state line has its state under the key with ".state" behind it
+        self.call_keys: List[List[Dict[str, Tuple[str, ...]]]] = []
         self.needs: Dict[str, object] = {}
         for st in spec.stages:
             keys = []
             for i, call in enumerate(st.calls):
                 base = call.cache or f"{st.name}.{i}"
-                mixers = spec.layers[call.layer].mixers()
+                cached = spec.layers[call.layer].cached_parts()
                 per_part = {}
-                for name, mixer in mixers:
-                    key = base if len(mixers) == 1 else f"{base}:{name}"
-                    need = part_class(mixer).cache_need(mixer.params)
-                    if call.writes_cache or key not in self.needs:
-                        if key in self.needs and self.needs[key] != need:
-                            raise ValueError(f"cache {key!r} is shared by layers that need different things: "
-                                             f"{self.needs[key]} and {need}")
-                        if need is not None:
-                            self.needs[key] = need
-                    per_part[name] = key
+                for name, part in cached:
+                    own = base if len(cached) == 1 else f"{base}:{name}"
+                    need = part_class(part).cache_need(part.params)
+                    several = need if isinstance(need, tuple) else (need,)
+                    if len(several) > 1 and sorted(type(n).__name__ for n in several) != ["PagedKvNeed", "StateNeed"]:
+                        raise ValueError(f"part {name!r} of {part.kind!r} keeps {several}: one set of pages and one state at most")
+                    keys_of_part = []
+                    for one in several:
+                        key = own + ".state" if len(several) > 1 and isinstance(one, StateNeed) else own
+                        if call.writes_cache or key not in self.needs:
+                            if key in self.needs and self.needs[key] != one:
+                                raise ValueError(f"cache {key!r} is shared by layers that need different things: "
+                                                 f"{self.needs[key]} and {one}")
+                            if one is not None:
+                                self.needs[key] = one
+                        keys_of_part.append(key)
+                    per_part[name] = tuple(keys_of_part)
                 keys.append(per_part)
             self.call_keys.append(keys)
         self.state_keys: List[Optional[str]] = []
@@ -99,14 +107,31 @@ class Model:
             plans.update(part.plan_rows(seq_rows, add, of[key]) if key in of else part.plan_rows(seq_rows, add))
         return plans
 
-    def _bind(self, ctx, key, cache):
-        need = self.needs.get(key)
-        if isinstance(need, PagedKvNeed):
-            ctx.group = cache.group_of[key]
-            ctx.plane = cache.groups[ctx.group].plane(key)
-            ctx.page_size = cache.page_size
-        elif isinstance(need, StateNeed):
-            ctx.state = cache.states[key]
+    def _bind(self, ctx, keys, cache):
+        for key in keys:
+            need = self.needs.get(key)
+            if isinstance(need, PagedKvNeed):
+                ctx.group = cache.group_of[key]
+                ctx.plane = cache.groups[ctx.group].plane(key)
+                ctx.page_size = cache.page_size
+            elif isinstance(need, StateNeed):
+                ctx.state = cache.states[key]
+        return ctx
+
+    def _call_context(self, j, i, b, cache):
+        """What call i of stage j sees of the step, with the caches that belong to it."""
+        st = self.spec.stages[j]
+        call, keys = st.calls[i], self.call_keys[j][i]
+        after = st.calls[i + 1].layer if i + 1 < len(st.calls) else None
+        # the rows going into a layer are replaced by its result: the layer may overwrite them
+        ctx = CallContext(batch=b, writes_cache=call.writes_cache, residual_is_spent=True,
+                          next_norm=getattr(self.layers[after], "first_norm", None) if after is not None
+                          else self.out_norms[j])
+        if len(keys) == 1:
+            self._bind(ctx, next(iter(keys.values())), cache)
+        elif keys:
+            ctx.bindings = {name: self._bind(CallContext(batch=b, writes_cache=call.writes_cache), of_part, cache)
+                            for name, of_part in keys.items()}
         return ctx
 
     def _run_stage(self, j, step, cache, prev):
@@ -114,19 +139,10 @@ class Model:
         state = cache.states.get(self.state_keys[j]) if self.state_keys[j] else None
         x = self.inputs[j].forward(b, prev, self.shared, state)
         if b.n_rows:
+            contexts = [self._call_context(j, i, b, cache) for i in range(len(st.calls))]
             for i, call in enumerate(st.calls):
-                keys = self.call_keys[j][i]
-                # the rows going into a layer are replaced by its result: the layer may overwrite them
-                after = st.calls[i + 1].layer if i + 1 < len(st.calls) else None
-                ctx = CallContext(batch=b, writes_cache=call.writes_cache, residual_is_spent=True,
-                                  next_norm=getattr(self.layers[after], "first_norm", None) if after is not None
-                                  else self.out_norms[j])
-                if len(keys) == 1:
-                    self._bind(ctx, next(iter(keys.values())), cache)
-                elif keys:
-                    ctx.bindings = {name: self._bind(CallContext(batch=b, writes_cache=call.writes_cache), key, cache)
-                                    for name, key in keys.items()}
-                x = self.layers[call.layer].forward(x, ctx)
+                contexts[i].next_call = contexts[i + 1] if i + 1 < len(contexts) else None
+                x = self.layers[call.layer].forward(x, contexts[i])
             x = self.out_norms[j](x)
         return x
 

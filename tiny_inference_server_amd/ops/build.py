@@ -48,6 +48,8 @@ SOURCES: Dict[str, str] = {
     "ssm_parts": "ssm_parts.hip",
     "delta_rule": "delta_rule.hip",
     "attention_mixed": "attention_mixed.hip",
+    "hyper_streams": "hyper_streams.hip",
+    "convolved_attention": "convolved_attention.hip",
 }
 HEADERS = ["common.h", "attention_mfma.h"]
 # what a library links beyond the HIP runtime

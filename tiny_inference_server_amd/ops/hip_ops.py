@@ -100,13 +100,13 @@ _SIGNATURES["attention_mfma"] = ("tis_attention_mfma", {
     "tis_attention_mfma": [_P, _L, _P, _P, _I, _P, _P, _P, _I, _I, _P, _I, _P, _L, _P, _P, _I, _I, _I, _I, _I, _I, _F,
                            _I, _I, _I, _I, _P, _P],
     "tis_attention_mfma_sink": [_P, _L, _P, _P, _I, _P, _P, _P, _I, _I, _P, _I, _P, _L, _P, _P, _I, _I, _I, _I, _I, _I, _F,
-                                _I, _I, _I, _I, _P, _I, _P],
+                                _I, _I, _I, _I, _P, _I, _P, _P],
 })
 
 _SIGNATURES["stream32"] = ("tis_stream32", {
     "tis_embed_scale": [_I, _P, _P, _F, _P, _P, _I, _I, _P],
     "tis_gated_postnorm": [_I, _P, _P, _L, _F, _P, _L, _F, _P, _L, _P, _F, _P, _F, _P, _P, _I, _I, _P],
-    "tis_rmsnorm32": [_I, _P, _P, _F, _P, _L, _I, _I, _P],
+    "tis_rmsnorm32": [_I, _P, _L, _P, _F, _P, _L, _I, _I, _P],
     "tis_head_norm_gate": [_I, _P, _L, _P, _L, _P, _I, _I, _F, _P, _L, _I, _I, _I, _P],
     "tis_lowrank_decay": [_P, _L, _I, _P, _P, _F, _P, _I, _I, _P],
     "tis_layernorm32": [_I, _P, _P, _P, _F, _P, _L, _I, _I, _P],
@@ -127,17 +127,18 @@ _SIGNATURES["stream32"] = ("tis_stream32", {
 _SIGNATURES["attention_window"] = ("tis_attention_window", {
     "tis_attention_prepare": [_I, _P, _L, _I, _I, _I, _P, _P, _P, _P, _L, _P, _P, _P, _P, _P, _P, _P, _I, _F, _I, _F, _I,
                               _I, _I, _I, _I, _I, _I, _I, _I, _P],
-    "tis_latent_prepare": [_I, _P, _L, _I, _I, _P, _P, _P, _P, _L, _P, _L, _P, _P, _I, _F, _I, _I, _I, _I, _I, _I, _P],
-    "tis_attention_window": [_I, _P, _L, _P, _P, _I, _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _L, _P],
+    "tis_latent_prepare": [_I, _P, _L, _I, _P, _L, _I, _P, _P, _P, _P, _L, _P, _L, _P, _P, _I, _I, _F, _F, _I, _I, _I, _I, _I, _I,
+                           _P],
+    "tis_attention_window": [_I, _P, _L, _P, _P, _I, _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _P, _L, _P, _P],
     "tis_attention_mixed": [_I, _P, _L, _P, _P, _I, _P, _P, _P, _L, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _F, _P, _P, _I, _P],
 })
 _SIGNATURES["attention_latent"] = ("tis_attention_latent", {
-    "tis_attention_latent": [_P, _L, _P, _P, _I, _P, _P, _P, _I, _P, _L, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P],
+    "tis_attention_latent": [_P, _L, _P, _P, _I, _P, _P, _P, _I, _P, _L, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I, _P, _P],
 })
 _SIGNATURES["experts"] = ("tis_experts", {
     "tis_route_topk": [_P, _L, _P, _F, _I, _I, _I, _I, _P, _P, _I, _I, _I, _P],
     "tis_expert_lists": [_P, _I, _I, _I, _P, _P, _P],
-    "tis_grouped_linear": [_I, _I, _P, _L, _L, _I, _P, _P, _L, _L, _P, _P, _I, _I, _I, _I, _I, _I, _P],
+    "tis_grouped_linear": [_I, _I, _P, _L, _L, _I, _P, _P, _L, _L, _P, _P, _I, _I, _I, _I, _I, _I, _P, _L, _P],
     "tis_experts_combine": [_I, _P, _L, _P, _L, _P, _P, _I, _I, _P, _L, _I, _I, _P],
 })
 _SIGNATURES["state_scan"] = ("tis_state_scan", {
@@ -157,6 +158,15 @@ _SIGNATURES["delta_rule"] = ("tis_delta_rule", {
 
 _SIGNATURES["attention_mixed"] = ("tis_attention_mixed", {
     "tis_attention_mixed_mfma": [_P, _L, _P, _P, _I, _P, _P, _P, _I, _P, _L, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _F, _P, _P, _P],
+})
+
+_SIGNATURES["hyper_streams"] = ("tis_hyper_streams", {
+    "tis_mix_streams": [_I, _P, _L, _L, _P, _L, _P, _P, _P, _P, _P, _P, _F, _P, _L, _P, _P, _L, _P, _P, _P, _I, _I, _I, _I, _P],
+})
+_SIGNATURES["convolved_attention"] = ("tis_convolved", {
+    "tis_convolved_prepare": [_I, _P, _L, _P, _P, _P, _L, _P, _P, _P, _P, _P, _P, _P, _L, _P, _I, _F, _P, _P, _I, _I, _I, _I, _I, _I,
+                              _I, _I, _P],
+    "tis_turn_back": [_I, _P, _L, _P, _I, _I, _I, _P],
 })
 
 _libs = {}
@@ -986,21 +996,24 @@ class HipOps:
                               f"{head_dim}] contiguous")
 
     def paged_attention(self, q, plane, batch, group, n_heads, n_kv_heads, head_dim, window=0, scale=None,
-                        slopes=None, sink=False, gate=None):
+                        slopes=None, sink=False, gate=None, turn=None):
         """Attention of the rows in `batch` over the cache plane; `q` is [rows, heads*head_dim] (a strided view is fine).
 
         `batch` brings positions, row_seq and the group's block tables; `group` names the page group. `slopes`
         ([heads] 32-bit, or None): a bias slope[h] * (key position - row position) on the scores; such calls go to
-        the general kernel. sink: the softmax's denominator also counts a key of score 0 that has no value. gate
-        ([rows, heads] 32-bit, a strided view is fine): head h's result is multiplied by sigmoid(gate[:, h]). Calls with
-        a sink or a gate that the matrix-core kernels do not take go to the kernel for keys and values of any sizes.
+        the general kernel. sink: the softmax's denominator also counts a key that has no value, of score 0 (True) or
+        sink[head] ([heads] 32-bit, not scaled). gate ([rows, heads] 32-bit, a strided view is fine): head h's result is
+        multiplied by sigmoid(gate[:, h]). turn ([rows, head_dim / 2, 2] 32-bit): the pairs (2m, 2m + 1) of every head's result
+        are turned back by the angle whose (cos, sin) is turn[row, m]. Calls with any of the three that the matrix-core
+        kernels do not take go to the kernel for keys and values of any sizes.
         window > 0: a row sees its last `window` keys; window < 0: the keys of its own chunk of -window positions, the
         chunks' edges at multiples of that size in the request (such calls, too, go to the kernel for any sizes where the matrix-core kernels do not
         take them); 0: all.
         """
         group_name = group
-        if (sink or gate is not None) and slopes is not None:
-            raise KernelError("attention: score slopes go with neither a sink nor a gate")
+        sink, sinks = self._sink(sink, n_heads)
+        if (sink or gate is not None or turn is not None) and slopes is not None:
+            raise KernelError("attention: score slopes go with neither a sink nor a gate nor turned values")
         _rows_view(self._check(q, "q"), "q")
         n = q.shape[0]
         page_size = plane.shape[3]
@@ -1102,20 +1115,47 @@ class HipOps:
                                         _ptr(batch.row_seq), _ptr(batch.positions), _ptr(items), n_items, nb, _ptr(tiles),
                                         n_tiles, _ptr(out), out.stride(0), _ptr(part_o), _ptr(part_ml), n, n_heads,
                                         n_kv_heads, head_dim, page_size, int(window), float(scale), n_splits, min_steps,
-                                        tile_splits, tile_max_steps, _ptr(row_splits), 1 if sink else 0, self._stream())
+                                        tile_splits, tile_max_steps, _ptr(row_splits), 1 if sink else 0, _ptr(sinks),
+                                        self._stream())
+            if turn is not None:
+                self.turn_back(out, turn, n_heads, head_dim)
             if gate is not None:
                 self.head_gate(out, gate, n_heads, head_dim)
             return out
-        if sink or gate is not None or window < 0:
+        if sink or gate is not None or turn is not None or window < 0:
             if slopes is not None:
                 raise KernelError("attention: score slopes do not go with chunks of positions")
             return self.paged_attention_kv(q, plane, batch, group_name, n_heads, n_kv_heads, head_dim, head_dim, page_size,
-                                           max(0, window), scale, sink=sink, gate=gate, chunk=max(0, -window))
+                                           max(0, window), scale, sink=sinks if sinks is not None else sink, gate=gate,
+                                           chunk=max(0, -window), turn=turn)
         self.attn_generic.tis_attention_generic(
             self.code, _ptr(q), q.stride(0), _ptr(plane), _ptr(tables), tables.stride(0), _ptr(batch.row_seq),
             _ptr(batch.positions), _ptr(out), out.stride(0), n, n_heads, n_kv_heads, head_dim, page_size, int(window),
             float(scale), _ptr(slopes), self._stream())
         return out
+
+    def _sink(self, sink, n_heads: int):
+        """(whether there is a sink, its scores per head or None for zeros) of a `sink` argument: False or None, True, or a
+        tensor of 32-bit scores."""
+        if torch.is_tensor(sink):
+            return True, self._f32(sink, "sink scores", n_heads)
+        return bool(sink), None
+
+    def _turn(self, turn, n: int, dim: int):
+        if dim % 2:
+            raise KernelError(f"attention: values of {dim} channels cannot be turned back in pairs")
+        return self._f32(turn, "angles of turned values", n * dim)
+
+    def turn_back(self, x, turn, n_heads: int, dim: int):
+        """In place: the pairs (2m, 2m + 1) of every head of x [rows, heads * dim] (compute type) are turned back by the
+        angle whose (cos, sin) is turn[row, m]; turn: [rows, dim / 2, 2] 32-bit."""
+        _rows_view(self._check(x, "turn_back x"), "turn_back x")
+        n = x.shape[0]
+        if x.shape[1] != n_heads * dim:
+            raise KernelError(f"turn_back: x {tuple(x.shape)} for {n_heads} heads of {dim}")
+        self._turn(turn, n, dim)
+        self._lazy("convolved_attention").tis_turn_back(self.code, _ptr(x), x.stride(0), _ptr(turn), n, n_heads, dim, self._stream())
+        return x
 
     # ---- a residual stream in 32-bit, norm after the sum ------------------------------------------------
     # The libraries below are loaded when a model first asks for them: a model that has no such part never
@@ -1178,12 +1218,12 @@ class HipOps:
         return out32, out
 
     def rmsnorm32(self, x32, gain, eps: float):
-        """x / sqrt(mean(x^2) + eps) * gain of 32-bit rows, in the compute type."""
+        """x / sqrt(mean(x^2) + eps) * gain of 32-bit rows (a strided view is fine), in the compute type."""
         n, D = x32.shape
-        self._f32(x32, "rmsnorm32 x", n * D)
+        self._f32_rows(x32, "rmsnorm32 x", n, D)
         self._f32(gain, "rmsnorm32 gain", D)
         out = self.empty(n, D)
-        self._lazy("stream32").tis_rmsnorm32(self.code, _ptr(x32), _ptr(gain), float(eps), _ptr(out), out.stride(0), n, D,
+        self._lazy("stream32").tis_rmsnorm32(self.code, _ptr(x32), x32.stride(0), _ptr(gain), float(eps), _ptr(out), out.stride(0), n, D,
                                              self._stream())
         return out
 
@@ -1531,19 +1571,20 @@ class HipOps:
         return out
 
     # ---- products in groups: experts, heads -----------------------------------------------------------------
-    def _grouped(self, a, lda, a_group, a_div, w, c, ldc, c_group, lists, counts, line, most_rows, act=0):
+    def _grouped(self, a, lda, a_group, a_div, w, c, ldc, c_group, lists, counts, line, most_rows, act=0, gate=None):
         G, N, K = w.shape
         self._check(w, "grouped product matrices")
         if not w.is_contiguous():
             raise KernelError("grouped product: the matrices must be contiguous [groups, out, in]")
         self._lazy("experts").tis_grouped_linear(
             _DT[a.dtype], _DT[c.dtype], _ptr(a), lda, a_group, a_div, _ptr(w), _ptr(c), ldc, c_group, _ptr(lists),
-            _ptr(counts), line, G, most_rows, N, K, act, self._stream())
+            _ptr(counts), line, G, most_rows, N, K, act, _ptr(gate), gate.stride(0) if gate is not None else 0, self._stream())
 
-    def heads_linear(self, x, w, out, out_group: int, out_offset: int = 0):
+    def heads_linear(self, x, w, out, out_group: int, out_offset: int = 0, gate=None):
         """A product per head on the head's own columns: out[:, out_offset + h * out_group + (0..N)] =
         x[:, h * K + (0..K)] . w[h]^T for w [heads, N, K]. x: [rows, heads * K] in the compute type; out: a 2-d tensor
-        of the compute type or 32-bit whose other columns are left as they are."""
+        of the compute type or 32-bit whose other columns are left as they are. gate ([rows, heads * N] 32-bit, a strided
+        view is fine): every result is multiplied by the sigmoid of its number."""
         _rows_view(self._check(x, "heads_linear x"), "heads_linear x")
         H, N, K = w.shape
         n = x.shape[0]
@@ -1555,8 +1596,10 @@ class HipOps:
         if out.shape[0] != n or out_offset < 0 or out_group < N or out_offset + (H - 1) * out_group + N > out.shape[1]:
             raise KernelError(f"heads_linear: out {tuple(out.shape)} for {n} rows, {H} heads of {N} every {out_group} from "
                               f"{out_offset}")
+        if gate is not None:
+            self._f32_rows(gate, "heads_linear gate", n, H * N)
         if n:
-            self._grouped(x, x.stride(0), K, 1, w, out[:, out_offset:], out.stride(0), out_group, None, None, 0, n)
+            self._grouped(x, x.stride(0), K, 1, w, out[:, out_offset:], out.stride(0), out_group, None, None, 0, n, gate=gate)
         return out
 
     def route_topk(self, z, correction, scale: float, top: int, score: str = "softmax", groups=None, renorm: bool = False):
@@ -1710,7 +1753,7 @@ class HipOps:
         return q
 
     def latent_prepare(self, proj, q_off, c_off, positions, write_slots, plane, n_heads, dim, rot_dim, rank, page_size,
-                       gain, freqs, rot_dims, eps, write_cache=True):
+                       gain, freqs, rot_dims, eps, write_cache=True, latent=None, pair_half=False, rot_factor: float = 1.0):
         """The step before attention over a shared latent. A row's 32-bit projections hold, from column q_off, its
         query heads as [dim unrotated | rot_dim rotated] each, and from c_off the latent (rank channels) followed by
         one rotated key part (rot_dim). Returns (q [rows, heads * (rank + rot_dim)] with every head's rotated part in
@@ -1718,9 +1761,13 @@ class HipOps:
         the compute type. The latent, RMS-normed with `gain`, and the rotated key part go into the pages at
         write_slots as keys of rank + rot_dim channels, and the latent once more as the key's value (pages of one
         key/value head with keys of rank + rot_dim and values of rank channels). Rotation: interleaved pairs of the
-        first rot_dims channels of the rotated parts, angle = position * freqs[pair]."""
+        first rot_dims channels of the rotated parts (pair_half: the pairs (i, i + rot_dims / 2)), angle = position *
+        freqs[pair], cosine and sine times rot_factor. latent: the 32-bit rows that c_off refers to, where they are not
+        proj itself."""
         n = proj.shape[0]
-        self._f32_rows(proj, "latent_prepare projections", n, max(q_off + n_heads * (dim + rot_dim), c_off + rank + rot_dim))
+        latent = proj if latent is None else latent
+        self._f32_rows(proj, "latent_prepare projections", n, q_off + n_heads * (dim + rot_dim))
+        self._f32_rows(latent, "latent_prepare latents", n, c_off + rank + rot_dim)
         self._index(positions, "positions", n)
         self._f32(gain, "latent norm gain", rank)
         if rot_dims:
@@ -1731,10 +1778,10 @@ class HipOps:
         q = self.empty(n, n_heads * (rank + rot_dim))
         q_plain = self.empty(n, n_heads * max(dim, 1))
         self._lazy("attention_window").tis_latent_prepare(
-            self.code, _ptr(proj), proj.stride(0), q_off, c_off, _ptr(positions), _ptr(write_slots if write_cache else None),
-            _ptr(plane if write_cache else None), _ptr(q), q.stride(0), _ptr(q_plain), q_plain.stride(0), _ptr(gain),
-            _ptr(freqs if rot_dims else None), int(rot_dims), float(eps), n, n_heads, dim, rot_dim, rank, page_size,
-            self._stream())
+            self.code, _ptr(proj), proj.stride(0), q_off, _ptr(latent), latent.stride(0), c_off, _ptr(positions),
+            _ptr(write_slots if write_cache else None), _ptr(plane if write_cache else None), _ptr(q), q.stride(0),
+            _ptr(q_plain), q_plain.stride(0), _ptr(gain), _ptr(freqs if rot_dims else None), int(rot_dims),
+            1 if pair_half else 0, float(rot_factor), float(eps), n, n_heads, dim, rot_dim, rank, page_size, self._stream())
         return q, q_plain
 
     def plan_latent(self, n_heads: int, seq_rows, add):
@@ -1745,16 +1792,20 @@ class HipOps:
         items = latent_items(seq_rows, n_heads)
         return {("latent_items", n_heads): (add(items), len(items))}
 
-    def latent_attention(self, q, plane, batch, group, n_heads, key_dim, value_dim, page_size, scale):
+    def latent_attention(self, q, plane, batch, group, n_heads, key_dim, value_dim, page_size, scale, window=0, sink=None):
         """Attention of the rows in `batch` over the pages of a latent: one key/value head, keys of key_dim channels
         whose first value_dim are also kept as values. q: [rows, heads * key_dim]; the result [rows, heads * value_dim].
+        window > 0: a row sees its last `window` keys. sink ([heads] 32-bit, or None): the softmax's denominator also counts
+        a key of score sink[head], not scaled, that has no value.
         bfloat16 with pages of 16 slots, key sizes in steps of 8 and value sizes in steps of 16 run on the matrix cores
         (a library per pair of sizes, compiled when first asked for); anything else on the kernel for any sizes."""
         _rows_view(self._check(q, "q"), "q")
         n = q.shape[0]
         if not (self.dtype == torch.bfloat16 and page_size == 16 and key_dim % 8 == 0 and value_dim % 16 == 0
                 and value_dim <= key_dim < 10000 and q.stride(0) % 8 == 0 and q.data_ptr() % 16 == 0):
-            return self.paged_attention_kv(q, plane, batch, group, n_heads, 1, key_dim, value_dim, page_size, 0, scale)
+            return self.paged_attention_kv(q, plane, batch, group, n_heads, 1, key_dim, value_dim, page_size, window, scale,
+                                           sink=sink)
+        _, sinks = self._sink(sink, n_heads)
         self._check_kv_plane(plane, 1, key_dim, value_dim, page_size)
         if q.shape[1] != n_heads * key_dim:
             raise KernelError(f"attention: q width {q.shape[1]} is not heads {n_heads} x key size {key_dim}")
@@ -1782,7 +1833,7 @@ class HipOps:
         # Portions: the four-wave kernel, every item's keys whole. Single rows: a wave per row and 16 heads, with
         # enough waves to fill the chip: a request's keys are cut where its rows alone would leave most units idle
         waves = n_items * -(-n_heads // 16)
-        steps = -(-batch.max_kv_len // 32)
+        steps = -(-(min(batch.max_kv_len, window + 31) if window else batch.max_kv_len) // 32)
         most = max(1, (self._workspace.numel() // (n * n_heads * (value_dim + 2))))
         # (a wave's step is two or three dependent trips to memory and little else, so many short chains beat few long
         # ones: four waves a compute unit, down to one step each)
@@ -1795,14 +1846,14 @@ class HipOps:
         lib.tis_attention_latent(_ptr(q), q.stride(0), _ptr(plane), _ptr(tables), tables.stride(0), _ptr(batch.row_seq),
                                  _ptr(batch.positions), _ptr(items), n_items, _ptr(out), out.stride(0), _ptr(part_o),
                                  _ptr(part_ml), n, n_heads, key_dim, value_dim, page_size, float(scale), n_splits,
-                                 self._stream())
+                                 int(window), _ptr(sinks), self._stream())
         return out
 
     def paged_attention_kv(self, q, plane, batch, group, n_heads, n_kv_heads, key_dim, value_dim, page_size, window=0,
-                           scale=None, sink=False, gate=None, chunk=0):
+                           scale=None, sink=False, gate=None, chunk=0, turn=None):
         """Attention of the rows in `batch` over pages whose keys have key_dim and whose values value_dim channels:
         [rows, heads*value_dim]. chunk > 0: a row at position p sees only the keys from p - p % chunk on (its own chunk
-        of positions; a chunk's edges are multiples of `chunk` in the request). sink: the softmax's denominator also counts a key of score 0 that has no value.
+        of positions; a chunk's edges are multiples of `chunk` in the request). sink, turn: as in paged_attention.
         gate: [rows, heads] 32-bit (a strided view is fine); head h's result is multiplied by sigmoid(gate[:, h])."""
         _rows_view(self._check(q, "q"), "q")
         n = q.shape[0]
@@ -1811,6 +1862,9 @@ class HipOps:
             raise KernelError(f"attention: q width {q.shape[1]} is not heads {n_heads} x key size {key_dim}")
         if gate is not None:
             self._f32_rows(gate, "attention gate", n, n_heads)
+        sink, sinks = self._sink(sink, n_heads)
+        if turn is not None:
+            self._turn(turn, n, value_dim)
         tables = batch.block_tables[group]
         self._check(tables, "block tables", torch.int32)
         if tables.dim() != 2 or tables.stride(1) != 1:
@@ -1824,9 +1878,105 @@ class HipOps:
         self._lazy("attention_window").tis_attention_window(
             self.code, _ptr(q), q.stride(0), _ptr(plane), _ptr(tables), tables.stride(0), _ptr(batch.row_seq),
             _ptr(batch.positions), _ptr(out), out.stride(0), n, n_heads, n_kv_heads, key_dim, value_dim, page_size,
-            int(window), int(chunk), float(scale if scale is not None else key_dim ** -0.5), 1 if sink else 0, _ptr(gate),
-            gate.stride(0) if gate is not None else 0, self._stream())
+            int(window), int(chunk), float(scale if scale is not None else key_dim ** -0.5), 1 if sink else 0, _ptr(sinks),
+            _ptr(gate), gate.stride(0) if gate is not None else 0, _ptr(turn), self._stream())
         return out
+
+    # ---- attention behind a short convolution, with values turned by position --------------------------------------
+    def convolved_prepare(self, proj, bias, taps, state, batch, write_slots, plane, n_heads, n_kv_heads, key_dim, value_dim,
+                          page_size, freqs, rot_dims, rot_factor, turn_freqs, write_cache=True):
+        """From a row's 32-bit projections (queries of all heads, keys, values side by side from column 0): the bias is
+        added, every channel passes a short convolution over the row and the rows before it (taps [channels, K], the last
+        column weighs the row itself; earlier rows come from the step's rows, and before those from the request's state
+        line, [K - 1, channels] 32-bit, oldest first, which is brought up to date), queries and keys are rotated in
+        interleaved pairs of their first rot_dims channels (angle = position * freqs[pair], cosine and sine times
+        rot_factor), values in interleaved pairs of all their channels by position * turn_freqs[pair] (None: not), and
+        keys and values go into the pages at write_slots. Returns (queries [rows, heads * key_dim] in the compute type,
+        (cos, sin) of the values' angles [rows, value_dim / 2, 2] 32-bit or None)."""
+        n = proj.shape[0]
+        C, K = taps.shape
+        if C != n_heads * key_dim + n_kv_heads * (key_dim + value_dim) or not write_cache:
+            raise KernelError(f"convolved_prepare: {C} channels for {n_heads} heads over {n_kv_heads}, keys of {key_dim}, values "
+                              f"of {value_dim}, write_cache={write_cache} (a cache that another call has written would bring "
+                              f"the state line forward twice)")
+        self._f32_rows(proj, "convolved_prepare projections", n, C)
+        self._f32(bias, "convolved_prepare bias", C)
+        self._f32(taps, "conv taps", C * K)
+        if rot_dims:
+            self._f32(freqs, "rotary frequencies", rot_dims // 2)
+        if turn_freqs is not None:
+            self._f32(turn_freqs, "values' frequencies", value_dim // 2)
+        if K > 1:
+            self._check_lines("convolved_prepare", state, (K - 1) * C, batch)
+        self._index(batch.row_seq, "row_seq", n)
+        self._index(batch.cu_rows, "cu_rows", batch.n_seqs + 1)
+        self._index(batch.seq_slots, "seq_slots", batch.n_seqs)
+        self._index(batch.positions, "positions", n)
+        self._index(write_slots, "write_slots", n)
+        self._check_kv_plane(plane, n_kv_heads, key_dim, value_dim, page_size)
+        q = self.empty(n, n_heads * key_dim)
+        turn = torch.empty(n, value_dim // 2, 2, dtype=torch.float32, device=self.device) if turn_freqs is not None else None
+        # rows a wave takes one after the other: with few rows one, so that a step still fills the chip
+        chunk = 1 if n <= 256 else 8
+        self._lazy("convolved_attention").tis_convolved_prepare(
+            self.code, _ptr(proj), proj.stride(0), _ptr(bias), _ptr(taps), _ptr(state if K > 1 else None),
+            state.stride(0) if K > 1 else 0, _ptr(batch.row_seq), _ptr(batch.cu_rows), _ptr(batch.seq_slots),
+            _ptr(batch.positions), _ptr(write_slots), _ptr(plane), _ptr(q), q.stride(0), _ptr(freqs if rot_dims else None),
+            int(rot_dims), float(rot_factor), _ptr(turn_freqs), _ptr(turn), n, K, n_heads, n_kv_heads, key_dim, value_dim,
+            page_size, chunk, self._stream())
+        return q, turn
+
+    # ---- a residual of several streams -------------------------------------------------------------------------------
+    def mix_streams(self, x, streams: int, write=None, read=None, shift=None):
+        """The end of one sublayer and the beginning of the next on a residual of `streams` 32-bit streams: (streams, rows).
+
+        x: [rows, streams, width], or [rows, width] where all streams are equal. write = (y, bias, mix, out): y ([rows, width]
+        32-bit, a strided view is fine) with its bias ([width] or None) joins, X_t <- sum_s mix[s, t] X_s + out[t] (y + bias);
+        the new streams come back (x itself without a write; with one, x may be overwritten). read = (weights, gain, eps):
+        rows in the compute type, the RMS norm of sum_t weights[t] X_t; else None. shift = (amount, state, batch): a row h
+        becomes h + (h_before - h) * amount with h_before the request's row before, which `state` ([slots, width] 32-bit)
+        keeps from step to step."""
+        n, D = x.shape[0], x.shape[-1]
+        S = int(streams)
+        if x.dim() == 3:
+            self._f32(x, "mix_streams x", n * S * D)
+            ldr, lds = S * D, D
+        else:
+            self._f32(x, "mix_streams x", n * D)
+            ldr, lds = D, 0
+        y = bias = mix = out = new = None
+        if write is not None:
+            y, bias, mix, out = write
+            self._f32_rows(y, "mix_streams y", n, D)
+            if bias is not None:
+                self._f32(bias, "mix_streams bias", D)
+            self._f32(mix, "stream mix", S * S)
+            self._f32(out, "stream factors", S)
+            # (a row before is worked out from the old streams again: they must stay)
+            new = x if x.dim() == 3 and shift is None else torch.empty(n, S, D, dtype=torch.float32, device=self.device)
+        h = weights = gain = amount = state = batch = None
+        eps = 0.0
+        if read is not None:
+            weights, gain, eps = read
+            self._f32(weights, "stream weights", S)
+            self._f32(gain, "mix_streams gain", D)
+            h = self.empty(n, D)
+        if shift is not None:
+            amount, state, batch = shift
+            self._f32(amount, "shift", D)
+            self._check_lines("mix_streams", state, D, batch)
+            self._index(batch.row_seq, "row_seq", n)
+            self._index(batch.cu_rows, "cu_rows", batch.n_seqs + 1)
+            self._index(batch.seq_slots, "seq_slots", batch.n_seqs)
+        # (rows that a workgroup takes in order: each such run works out one row before again)
+        chunk = 4 if shift is not None and n > 1024 else 1
+        self._lazy("hyper_streams").tis_mix_streams(
+            self.code, _ptr(x), ldr, lds, _ptr(y), y.stride(0) if y is not None else 0, _ptr(bias), _ptr(mix), _ptr(out),
+            _ptr(new), _ptr(weights), _ptr(gain), float(eps), _ptr(h), h.stride(0) if h is not None else 0, _ptr(amount),
+            _ptr(state), state.stride(0) if state is not None else 0, _ptr(batch.row_seq if batch is not None else None),
+            _ptr(batch.cu_rows if batch is not None else None), _ptr(batch.seq_slots if batch is not None else None), n, D, S,
+            chunk, self._stream())
+        return (new if write is not None else x), h
 
     def plan_row_tiles(self, seq_rows, add):
         """Host planning for the matrix-core attention with mixed sigmoid weights: its items for a step's rows, (first

@@ -4,7 +4,7 @@ from __future__ import annotations
 import torch
 
 from .base import MIXERS, build_part, to_compute
-from .spec import PagedKvNeed
+from .spec import PagedKvNeed, StateNeed
 
 
 @MIXERS.register("gqa_attention")
@@ -199,6 +199,42 @@ def _rotary_frequencies(ops, dims: int, base: float, bands=None):
     return banded_frequencies(dims, base, bands).to(torch.float32).to(ops.device)
 
 
+def slowed_frequencies(dims: int, base: float, factor: float, original: float, fast: float, slow: float):
+    """(frequencies in 64-bit, factor on cosine and sine) of a rotation whose long waves are slowed by `factor`.
+
+    A pair that turns n times within `original` positions sits at i(n) = dims ln(original / (2 pi n)) / (2 ln base). Up to
+    pair floor(i(fast)) the frequencies base^(-2i/dims) are kept, from pair ceil(i(slow)) on they are divided by `factor`,
+    and linearly blended between the two (both clamped to 0 .. dims - 1; where they coincide, a step)."""
+    import math
+    f = banded_frequencies(dims, base)
+    at = [dims * math.log(original / (2.0 * math.pi * n)) / (2.0 * math.log(base)) for n in (fast, slow)]
+    lo, hi = max(math.floor(at[0]), 0), min(math.ceil(at[1]), dims - 1)
+    ramp = torch.clamp((torch.arange(dims // 2, dtype=torch.float64) - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return f / factor * ramp + f * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
+
+
+def _rotation(ops, dims: int, base: float, slowed=None):
+    """(frequencies on the device in 32-bit, factor on cosine and sine); slowed: (factor, original, fast, slow) or None."""
+    if slowed is None or not dims:
+        return _rotary_frequencies(ops, dims, base), 1.0
+    f, factor = slowed_frequencies(dims, base, *(float(v) for v in slowed))
+    return f.to(torch.float32).to(ops.device), factor
+
+
+def stacked_rows(mats):
+    """(the matrices one below the other, each starting at a multiple of 8 rows; their first rows): the columns of a
+    32-bit product with them then start 32 bytes apart."""
+    blocks, starts, at = [], [], 0
+    for m in mats:
+        pad = -m.shape[0] % 8
+        starts.append(at)
+        blocks.append(m)
+        if pad:
+            blocks.append(torch.zeros(pad, m.shape[1], dtype=m.dtype, device=m.device))
+        at += m.shape[0] + pad
+    return torch.cat(blocks, dim=0), starts
+
+
 @MIXERS.register("sink_gated_attention")
 class SinkGatedAttention:
     """Grouped-query attention over all earlier positions with biased projections, no rotation, a query factor that
@@ -287,11 +323,14 @@ class SinkGatedAttention:
 class LatentAttention:
     """Softmax attention whose keys and values are made from one low-rank latent per position.
 
-    q = x.Wq^T, a head being [dim unrotated | rot_dim rotated] channels. x.Wdkv^T gives rank + rot_dim channels: the
-    first rank, RMS-normed with a gain, are the latent c; the others are one rotated key part that all heads share.
-    Head h's unrotated key is Wuk[h] c and its value Wuv[h] c; score = (q_plain . k_plain + q_rot . k_rot) * scale;
-    rotation in interleaved pairs of the first rot_dims channels of the rotated parts by position * base^(-2i/rot_dims);
-    causal softmax; out = heads . Wo^T.
+    q = x.Wq^T, a head being [dim unrotated | rot_dim rotated] channels; with q_rank > 0 the queries go through a latent
+    of their own, q = rmsnorm(x.Wdq^T).Wuq^T. x.Wdkv^T gives rank + rot_dim channels: the first rank, RMS-normed with a
+    gain, are the latent c; the others are one rotated key part that all heads share. Head h's unrotated key is Wuk[h] c
+    and its value Wuv[h] c; score = (q_plain . k_plain + q_rot . k_rot) * scale; rotation of the first rot_dims channels of
+    the rotated parts in interleaved pairs (pair_half: in the pairs (i, i + rot_dims / 2)) by position * base^(-2i/rot_dims),
+    or by the frequencies and with the factor of `slowed_frequencies` (rot_slowed); causal softmax over all earlier
+    positions or the last `window`, with a learned sink per head (sink: one more key of score sink[h], not scaled, without
+    a value); the heads side by side are multiplied by sigmoid(x.Wg^T) channel by channel (gate); out = heads . Wo^T.
 
     Only c and the rotated key part are kept, as one key of rank + rot_dim channels per position whose value is c
     again (transposed, as the attention kernels read values). The products with
@@ -299,35 +338,52 @@ class LatentAttention:
     query becomes [Wuk[h]^T q_plain | q_rot] against the key [c | k_rot]; and sum_j p_j Wuv[h] c_j = Wuv[h] sum_j p_j c_j,
     so the attention's values are the latents themselves and Wuv[h] is applied to the result.
 
-    params: width, n_heads, dim, rot_dim, value_dim, rank, rot_dims, rot_base, scale, eps. tensors, stored [out, in]:
-    q (heads*(dim+rot_dim), width), dkv (rank+rot_dim, width), dkv_norm (rank,), uk (heads*dim, rank),
-    uv (heads*value_dim, rank), o (width, heads*value_dim).
+    params: width, n_heads, dim, rot_dim, value_dim, rank, rot_dims, rot_base, scale, eps, and optionally q_rank (0),
+    window (0: all), pair_half, rot_slowed, sink, gate. tensors, stored [out, in]: q (heads*(dim+rot_dim), width), or with
+    q_rank dq (q_rank, width), dq_norm (q_rank,), uq (heads*(dim+rot_dim), q_rank); dkv (rank+rot_dim, width), dkv_norm
+    (rank,), uk (heads*dim, rank), uv (heads*value_dim, rank), o (width, heads*value_dim), with sink: sink (heads,), with
+    gate: gate (heads*value_dim, width).
     """
     graph_safe = True
 
     @classmethod
     def tensor_shapes(cls, params):
         w, H, D, R, V, C = (params[k] for k in ("width", "n_heads", "dim", "rot_dim", "value_dim", "rank"))
-        return {"q": (H * (D + R), w), "dkv": (C + R, w), "dkv_norm": (C,), "uk": (H * D, C), "uv": (H * V, C),
-                "o": (w, H * V)}
+        Q = params.get("q_rank", 0)
+        shapes = {"dq": (Q, w), "dq_norm": (Q,), "uq": (H * (D + R), Q)} if Q else {"q": (H * (D + R), w)}
+        shapes.update({"dkv": (C + R, w), "dkv_norm": (C,), "uk": (H * D, C), "uv": (H * V, C), "o": (w, H * V)})
+        if params.get("sink", False):
+            shapes["sink"] = (H,)
+        if params.get("gate", False):
+            shapes["gate"] = (H * V, w)
+        return shapes
 
     @classmethod
     def cache_need(cls, params):
-        return PagedKvNeed(1, params["rank"] + params["rot_dim"], 0, value_dim=params["rank"])
+        return PagedKvNeed(1, params["rank"] + params["rot_dim"], int(params.get("window", 0)), value_dim=params["rank"])
 
     def __init__(self, spec, tensors, ops):
         from .base import to_gain
         p = spec.params
         self.ops = ops
         self.H, self.D, self.R, self.V, self.C = (int(p[k]) for k in ("n_heads", "dim", "rot_dim", "value_dim", "rank"))
-        self.rot_dims = int(p.get("rot_dims", self.R))
+        self.q_rank, self.window = int(p.get("q_rank", 0)), int(p.get("window", 0))
+        self.rot_dims, self.pair_half = int(p.get("rot_dims", self.R)), bool(p.get("pair_half", False))
         if self.rot_dims % 2 or self.rot_dims > self.R:
             raise ValueError(f"{self.rot_dims} rotated channels of a part of {self.R}: an even number, at most the part")
         self.scale, self.eps = float(p["scale"]), float(p["eps"])
-        self.freqs = _rotary_frequencies(ops, self.rot_dims, float(p.get("rot_base", 10000.0)))
-        wq, wdkv = tensors.of(spec, "q"), tensors.of(spec, "dkv")
-        self.c_at = wq.shape[0]
-        self.w_in = to_compute(ops, torch.cat((wq, wdkv), dim=0))
+        self.freqs, self.rot_factor = _rotation(ops, self.rot_dims, float(p.get("rot_base", 10000.0)), p.get("rot_slowed"))
+        # one product for everything that reads the row; every block of it starts at a multiple of 8 rows
+        mats = [tensors.of(spec, "dq" if self.q_rank else "q"), tensors.of(spec, "dkv")]
+        if p.get("gate", False):
+            mats.append(tensors.of(spec, "gate"))
+        w_in, starts = stacked_rows(mats)
+        self.c_at, self.g_at = starts[1], starts[2] if len(mats) > 2 else None
+        self.w_in = to_compute(ops, w_in)
+        if self.q_rank:
+            self.q_gain = to_gain(ops, tensors.of(spec, "dq_norm"))
+            self.w_uq = to_compute(ops, tensors.of(spec, "uq"))
+        self.sink = to_gain(ops, tensors.of(spec, "sink")) if p.get("sink", False) else None
         self.c_gain = to_gain(ops, tensors.of(spec, "dkv_norm"))
         # [heads, rank, dim]: Wuk[h]^T, which takes a head's unrotated query into the latent's space
         self.w_uk_t = to_compute(ops, tensors.of(spec, "uk").view(self.H, self.D, self.C).transpose(1, 2))
@@ -345,17 +401,125 @@ class LatentAttention:
         ops, b = self.ops, ctx.batch
         H, D, R, V, C = self.H, self.D, self.R, self.V, self.C
         proj = ops.linear(x, self.w_in, out_dtype=torch.float32)
-        q, q_plain = ops.latent_prepare(proj, 0, self.c_at, b.positions, b.write_slots[ctx.group], ctx.plane, H, D, R, C,
-                                        ctx.page_size, self.c_gain, self.freqs, self.rot_dims, self.eps, ctx.writes_cache)
+        queries = proj
+        if self.q_rank:
+            queries = ops.linear(ops.rmsnorm32(proj[:, :self.q_rank], self.q_gain, self.eps), self.w_uq, out_dtype=torch.float32)
+        q, q_plain = ops.latent_prepare(queries, 0, self.c_at, b.positions, b.write_slots[ctx.group], ctx.plane, H, D, R, C,
+                                        ctx.page_size, self.c_gain, self.freqs, self.rot_dims, self.eps, ctx.writes_cache,
+                                        latent=proj, pair_half=self.pair_half, rot_factor=self.rot_factor)
         ops.heads_linear(q_plain, self.w_uk_t, q, C + R)
-        mixed = ops.latent_attention(q, ctx.plane, b, ctx.group, H, C + R, C, ctx.page_size, self.scale)
-        return ops.heads_linear(mixed, self.w_uv, ops.empty(mixed.shape[0], H * V), V)
+        mixed = ops.latent_attention(q, ctx.plane, b, ctx.group, H, C + R, C, ctx.page_size, self.scale, window=self.window,
+                                     sink=self.sink)
+        gate = proj[:, self.g_at:self.g_at + H * V] if self.g_at is not None else None
+        return ops.heads_linear(mixed, self.w_uv, ops.empty(mixed.shape[0], H * V), V, gate=gate)
 
     def forward32(self, x, ctx):
         return self.ops.linear(self.core(x, ctx), self.w_o, out_dtype=torch.float32)
 
     def forward(self, x, ctx, residual=None):
         return self.ops.linear(self.core(x, ctx), self.w_o, residual=residual)
+
+
+@MIXERS.register("convolved_attention")
+class ConvolvedAttention:
+    """Grouped-query softmax attention whose queries, keys and values pass a short convolution over time, with keys and
+    values turned by their position and a learned sink.
+
+    q = x.Wq^T + bq, k = x.Wk^T + bk, v = x.Wv^T + bv; then, channel by channel, y_t = sum_d taps[K-1-d] u_(t-d) over the row
+    and the K - 1 rows before it (nothing before a request's first row). The first rot_dims channels of every query and key
+    head are rotated in interleaved pairs by position * base^(-2i/rot_dims), or by the frequencies and with the factor of
+    `slowed_frequencies` (rot_slowed). Values are turned over all their channels in interleaved pairs by position *
+    turn_base^(-2m/value_dim) and cached so; a head's result at position p is turned back by p (turn_base None: values
+    are left as they are). score = q.k * scale; causal softmax over all earlier positions or the last `window` with one
+    more key of score sink[h], not scaled, without a value; out = heads . Wo^T + bo. Convolution, angles, scores and the
+    softmax are 32-bit.
+
+    The pages hold turned keys and values; a state line per request holds the last taps - 1 projected rows [taps - 1,
+    heads*key_dim + kv_heads*(key_dim + value_dim)], oldest first.
+
+    params: width, n_heads, n_kv_heads, key_dim, value_dim, taps, scale, rot_dims, rot_base, rot_slowed, turn_base, window.
+    tensors, stored [out, in]: q (heads*key_dim, width), k (kv_heads*key_dim, width), v (kv_heads*value_dim, width), q_bias,
+    k_bias, v_bias, q_conv, k_conv, v_conv ([channels, taps], the last column weighs the row itself), sink (heads,),
+    o (width, heads*value_dim), o_bias (width,).
+    """
+    graph_safe = True
+
+    @classmethod
+    def tensor_shapes(cls, params):
+        w, H, G, kd, vd, K = (params[k] for k in ("width", "n_heads", "n_kv_heads", "key_dim", "value_dim", "taps"))
+        shapes = {"sink": (H,), "o": (w, H * vd), "o_bias": (w,)}
+        for name, channels in (("q", H * kd), ("k", G * kd), ("v", G * vd)):
+            shapes.update({name: (channels, w), name + "_bias": (channels,), name + "_conv": (channels, K)})
+        return shapes
+
+    @classmethod
+    def cache_need(cls, params):
+        H, G, kd, vd, K = (params[k] for k in ("n_heads", "n_kv_heads", "key_dim", "value_dim", "taps"))
+        pages = PagedKvNeed(G, kd, int(params.get("window", 0)), value_dim=vd)
+        floats = (K - 1) * (H * kd + G * (kd + vd))
+        return (pages, StateNeed((floats,), "float32")) if floats else pages
+
+    def __init__(self, spec, tensors, ops):
+        from .base import to_gain
+        p = spec.params
+        self.ops = ops
+        self.H, self.G, self.kd, self.vd, self.K = (int(p[k]) for k in ("n_heads", "n_kv_heads", "key_dim", "value_dim", "taps"))
+        if self.H % self.G:
+            raise ValueError(f"{self.H} query heads are not a multiple of {self.G} key/value heads")
+        self.scale, self.window = float(p["scale"]), int(p.get("window", 0))
+        self.rot_dims = int(p.get("rot_dims", 0))
+        if self.rot_dims % 2 or self.rot_dims > self.kd:
+            raise ValueError(f"{self.rot_dims} rotated channels of a head of {self.kd}: an even number, at most the head")
+        self.freqs, self.rot_factor = _rotation(ops, self.rot_dims, float(p.get("rot_base", 10000.0)), p.get("rot_slowed"))
+        turn = p.get("turn_base")
+        if turn is not None and self.vd % 2:
+            raise ValueError(f"values of {self.vd} channels cannot be turned in pairs")
+        self.turn_freqs = _rotary_frequencies(ops, self.vd, float(turn)) if turn is not None else None
+        self.w_in = to_compute(ops, torch.cat([tensors.of(spec, k) for k in ("q", "k", "v")], dim=0))
+        self.bias = to_gain(ops, torch.cat([tensors.of(spec, k + "_bias") for k in ("q", "k", "v")], dim=0))
+        self.taps = to_gain(ops, torch.cat([tensors.of(spec, k + "_conv") for k in ("q", "k", "v")], dim=0))
+        self.sink, self.o_bias = to_gain(ops, tensors.of(spec, "sink")), to_gain(ops, tensors.of(spec, "o_bias"))
+        self.w_o = to_compute(ops, tensors.of(spec, "o"))
+        self.same = self.kd == self.vd        # then the pages have the layout every attention kernel reads
+
+    # the matrix-core kernels' work lists, where keys and values are of one size (see GqaAttention)
+    def plan_key(self):
+        if not self.same or not hasattr(self.ops, "plan_attention"):
+            return None
+        return ("attention", self.H, self.G, self.kd, self.window)
+
+    def plan_mode(self, seq_rows):
+        mode = getattr(self.ops, "plan_attention_mode", None)
+        return mode(seq_rows, self.window) if mode is not None and self.same else None
+
+    def plan_rows(self, seq_rows, add, mode=None):
+        return self.ops.plan_attention(self.H, self.G, self.kd, seq_rows, add, mode, self.window)
+
+    def core(self, x, ctx):
+        ops, b = self.ops, ctx.batch
+        proj = ops.linear(x, self.w_in, out_dtype=torch.float32)
+        q, turn = ops.convolved_prepare(proj, self.bias, self.taps, ctx.state, b, b.write_slots[ctx.group], ctx.plane, self.H,
+                                        self.G, self.kd, self.vd, ctx.page_size, self.freqs, self.rot_dims, self.rot_factor,
+                                        self.turn_freqs, ctx.writes_cache)
+        if self.same:
+            return ops.paged_attention(q, ctx.plane, b, ctx.group, self.H, self.G, self.kd, self.window, self.scale,
+                                       sink=self.sink, turn=turn)
+        return ops.paged_attention_kv(q, ctx.plane, b, ctx.group, self.H, self.G, self.kd, self.vd, ctx.page_size, self.window,
+                                      self.scale, sink=self.sink, turn=turn)
+
+    def forward_parts(self, x, ctx):
+        """(the result without its output bias, 32-bit; the bias): for a block whose sum adds the bias."""
+        return self.ops.linear(self.core(x, ctx), self.w_o, out_dtype=torch.float32), self.o_bias
+
+    def forward32(self, x, ctx):
+        y, bias = self.forward_parts(x, ctx)
+        return y + bias
+
+    def forward(self, x, ctx, residual=None):
+        y = self.forward32(x, ctx)
+        if residual is not None:
+            y = y + residual.to(torch.float32)
+        return y.to(self.ops.dtype)
 
 
 @MIXERS.register("chunked_attention")

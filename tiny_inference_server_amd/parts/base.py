@@ -20,7 +20,8 @@ every part      graph_safe = True                      class attribute, only if 
                                                        as graphs); absent or False keeps the model on plain launches;
                                                        "single_rows": the promise holds for steps in which every
                                                        request brings one token (those are still captured)
-mixer           cache_need(params) -> PagedKvNeed | StateNeed | None      classmethod
+mixer           cache_need(params) -> PagedKvNeed | StateNeed | None, or a tuple of one PagedKvNeed and one StateNeed for
+                                                       a mixer that keeps both      classmethod
                 forward(x, ctx, residual=None) -> y    x: normed rows; ctx: CallContext; adds `residual` if given
 feed-forward    forward(x, residual=None) -> y
                 a mixer or feed-forward with the class attribute fuses_norm = True takes forward(..., norm=part)
@@ -33,6 +34,8 @@ planning        a part may offer plan_key() -> hashable | None and plan_rows(seq
                 step's arrays are packed, found again in batch.extras[name]
 token input     forward(x, tokens) -> (y, norm | None): what a block adds to its stream from a table indexed by the rows'
                 tokens; x is the stream in the compute type, y 32-bit, norm = (gain, eps) if y is still to be RMS-normed
+connection      how a sublayer's result joins a residual of several streams: mix, out (32-bit tensors); see parts/hyper32.py
+row shift       cache_need(params) like a mixer; what a mixer reads is mixed with the row before it: amount (32-bit tensor)
 stage input     state_need(params) -> StateNeed | None classmethod
                 forward(batch, previous_output, previous_batch, shared, state) -> rows
 """
@@ -51,14 +54,16 @@ ARRANGEMENTS: Registry = Registry("block arrangement")
 STAGE_INPUTS: Registry = Registry("stage input")
 GATES: Registry = Registry("residual gate")
 TOKEN_INPUTS: Registry = Registry("per-layer token input")
+CONNECTIONS: Registry = Registry("stream connection")
+ROW_SHIFTS: Registry = Registry("row shift")
 
 
 @dataclass
 class CallContext:
     """What one layer call sees of the step: the rows' metadata and the cache that belongs to the call.
 
-    A block with one mixer finds that mixer's cache right here. A block with several asks `ctx.of(part name)` for
-    each mixer's own context (same batch, that part's cache)."""
+    A block with one mixer finds that mixer's cache right here. A block with several parts that keep something asks
+    `ctx.of(part name)` for each part's own context (same batch, that part's cache)."""
     batch: Any                       # engine.batch.StageBatch
     group: Optional[str] = None      # page group of the call's cache, for paged needs
     plane: Any = None                # [pages, 2, kv heads, page size, head size] for paged needs (keys and values of
@@ -70,6 +75,8 @@ class CallContext:
     next_norm: Any = None            # the norm part that reads this call's result next (the following block's first
                                      # norm, as it says in `first_norm`, or the stage's closing norm), if known: a block
                                      # may fuse it into its last kernel
+    next_call: Optional["CallContext"] = None    # that following call's own context (None: the stage ends here), for what a
+                                     # fused norm keeps between steps
     bindings: Optional[Dict[str, "CallContext"]] = None     # per mixer part of the block
 
     def of(self, part_name: str) -> "CallContext":
@@ -108,7 +115,8 @@ class Tensors:
 
 
 REGISTRIES = {"mixer": MIXERS, "feed_forward": FEED_FORWARDS, "norm": NORMS, "position": POSITION_ENCODINGS,
-              "stage_input": STAGE_INPUTS, "gate": GATES, "token_input": TOKEN_INPUTS}
+              "stage_input": STAGE_INPUTS, "gate": GATES, "token_input": TOKEN_INPUTS, "connection": CONNECTIONS,
+              "row_shift": ROW_SHIFTS}
 
 
 def part_class(spec):

@@ -21,17 +21,22 @@ from typing import Any, Mapping, Optional, Tuple
 @dataclass(frozen=True)
 class PartSpec:
     role: str                     # which registry `kind` is looked up in: "norm", "position", "mixer",
-                                  # "feed_forward", "gate", "token_input" or "stage_input"
+                                  # "feed_forward", "gate", "token_input", "connection", "row_shift" or "stage_input"
     kind: str
     params: Mapping[str, Any] = field(default_factory=dict)    # sizes, constants, nested PartSpecs
     tensors: Mapping[str, str] = field(default_factory=dict)   # local key -> tensor name in the file
+
+
+# the roles whose parts may ask for a cache of their own (pages, a state line per request, or both)
+CACHED_ROLES = ("mixer", "row_shift")
 
 
 @dataclass(frozen=True)
 class LayerSpec:
     """One block. Which parts a block has is the arrangement's business: it declares their names, and the loader,
     the cache manager and the graph check walk whatever is there. A block may have no feed-forward, two mixers,
-    norms in other places; every part whose role is "mixer" gets a cache of its own if its kind asks for one."""
+    norms in other places; every part whose role is one of CACHED_ROLES gets a cache of its own if its kind asks for
+    one."""
     arrangement: str                      # block arrangement kind, e.g. "prenorm_residual"
     parts: Mapping[str, PartSpec]         # the arrangement's name for the part -> the part
     params: Mapping[str, Any] = field(default_factory=dict)    # the arrangement's own constants
@@ -47,6 +52,9 @@ class LayerSpec:
 
     def mixers(self) -> Tuple[Tuple[str, PartSpec], ...]:
         return tuple((n, p) for n, p in self.parts.items() if p.role == "mixer")
+
+    def cached_parts(self) -> Tuple[Tuple[str, PartSpec], ...]:
+        return tuple((n, p) for n, p in self.parts.items() if p.role in CACHED_ROLES)
 
 
 @dataclass(frozen=True)
