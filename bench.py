@@ -359,6 +359,21 @@ def fesupel_config(width, heads, kv_heads, ff, layers, vocab, experts=8, top=2, 
                                         for i in range(layers)]})
 
 
+def gosavik_config(width, heads, kv_heads, ff, layers, vocab, window=1024, streams=4):
+    """Attention over a latent inside a window and convolved attention with turned values in turn, a dense feed-forward, a
+    residual of `streams` streams; no layer is passed twice."""
+    from tiny_inference_server_amd.config import config_from_dict
+    dense = {"kind": "dense", "ff": ff}
+    latent = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "q_rank": 3 * width // 4,
+              "scale": 192 ** -0.5, "mask": {"size": window},
+              "rot": {"dims": 64, "base": 10000.0, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    att = {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "conv": 4, "scale": 128 ** -0.5,
+           "rot": {"dims": 128, "base": 500000.0}}
+    kinds = [("latent_attention", latent), ("attention", att)]
+    return config_from_dict({"architecture": "Gosavik", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "streams": streams,
+                             "layers": [{"type": t, "mixer": m, "mlp": dense} for t, m in (kinds[i % 2] for i in range(layers))]})
+
+
 def design_comparison(a, say):
     """Prefill (a.prefill_tokens tokens, one prompt) and decode (batch a.batch, context a.context) of the Fikevik and
     Fipuzen designs and of the grouped-query decoder without prediction heads at the sizes of DESIGN_SIZES, random
@@ -381,6 +396,7 @@ def design_comparison(a, say):
             "fipuzen": fipuzen_config(width, heads, kv_heads, ff, layers, vocab),
             "rurorax": rurorax_config(width, heads, kv_heads, ff, layers, vocab),
             "fesupel": fesupel_config(width, heads, kv_heads, ff, layers, vocab),
+            "gosavik": gosavik_config(width, heads, kv_heads, ff, layers, vocab),
             "gqa": GqaMtpConfig(d_model=width, vocab_size=vocab, max_context=max(8192, a.context), rope_base=500000.0,
                                 n_heads=heads, n_layers=layers, ffn_hidden=ff, group_size=heads // kv_heads, mtp_heads=0,
                                 rms_eps=1e-5, tie_embeddings=False),
@@ -439,7 +455,7 @@ def design_comparison(a, say):
             "warmup": a.warmup, "ms_per_step": points[first].get("decode_ms"), "higher_is_better": True,
             "scaling": "weak", "vs_baseline": None, "dtype": dkey,
             "data": "synthetic: random weights N(0,0.02), uniform random token ids",
-            "config": {"model": "Fikevik, Fipuzen, Rurorax and Fesupel beside GqaMtpTransformer", "sizes": [list(s) for s in DESIGN_SIZES],
+            "config": {"model": "Fikevik, Fipuzen, Rurorax, Fesupel and Gosavik beside GqaMtpTransformer", "sizes": [list(s) for s in DESIGN_SIZES],
                        "global_batch": a.batch, "seq_len": a.context, "prefill_tokens": a.prefill_tokens,
                        "parallelism": "single-gpu"},
             "points": points}
@@ -467,7 +483,7 @@ def main() -> int:
     ap.add_argument("--seed", type=int, default=0)
     ap.add_argument("--workload", choices=["decode", "serve", "mixed", "designs"], default="decode")
     ap.add_argument("--requests", type=int, default=64, help="serve, mixed: requests (decoding at once)")
-    ap.add_argument("--designs", default="", help="designs: which of fikevik,fipuzen,rurorax,fesupel,gqa to run (default: all)")
+    ap.add_argument("--designs", default="", help="designs: which of fikevik,fipuzen,rurorax,fesupel,gosavik,gqa to run (default: all)")
     ap.add_argument("--design-sizes", default="", help="designs: which sizes to run, e.g. w2048 (default: all)")
     ap.add_argument("--phase", choices=["both", "prefill", "decode"], default="both", help="designs: what to measure")
     ap.add_argument("--new-tokens", type=int, default=256, help="serve: tokens generated per request")
