@@ -207,7 +207,7 @@ __global__ __launch_bounds__(MS_THREADS) void mix_streams_any_kernel(MixArgs a) 
   }
 }
 
-// x_new must not overlap x where there is a row before (amount), and may be x itself where there is none.
+// x_new must not overlap x: old streams are read again for a row before, and where sizes are not the usual ones.
 TIS_EXPORT int tis_mix_streams(int dtype, const float* x, long ldr, long lds, const float* y, long ldy, const float* y_bias,
                                const float* mix, const float* out, float* x_new, const float* read, const float* gain,
                                float eps, void* h, long ldh, const float* amount, float* state, long state_ld,
@@ -218,8 +218,9 @@ TIS_EXPORT int tis_mix_streams(int dtype, const float* x, long ldr, long lds, co
     return tis_fail("mix_streams: bad arguments rows=%d width=%d streams=%d", rows, D, S);
   if (y && (!mix || !out || !x_new)) return tis_fail("mix_streams: a result that joins needs a mix, factors and new streams");
   if (h && (!read || !gain)) return tis_fail("mix_streams: a norm needs the streams' weights and a gain");
-  if (amount && (!h || !state || !row_seq || !cu_rows || !seq_slots || state_ld < D || (y && x == x_new)))
-    return tis_fail("mix_streams: a row before needs its norm, kept rows of %d, the rows' requests, and new streams of their own", D);
+  if (y && x == x_new) return tis_fail("mix_streams: the new streams need memory of their own");
+  if (amount && (!h || !state || !row_seq || !cu_rows || !seq_slots || state_ld < D))
+    return tis_fail("mix_streams: a row before needs its norm, kept rows of %d and the rows' requests", D);
   const MixArgs a{x, ldr, lds, y, ldy, y_bias, mix, out, x_new, read, gain, eps, h, ldh, amount, state, state_ld, row_seq,
                   cu_rows, seq_slots, rows, D, S, chunk};
   if (dtype != TIS_F32 && dtype != TIS_BF16) return tis_fail("unknown dtype code %d", dtype);

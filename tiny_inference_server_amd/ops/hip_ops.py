@@ -1932,7 +1932,7 @@ class HipOps:
 
         x: [rows, streams, width], or [rows, width] where all streams are equal. write = (y, bias, mix, out): y ([rows, width]
         32-bit, a strided view is fine) with its bias ([width] or None) joins, X_t <- sum_s mix[s, t] X_s + out[t] (y + bias);
-        the new streams come back (x itself without a write; with one, x may be overwritten). read = (weights, gain, eps):
+        the new streams come back in memory of their own (x itself without a write). read = (weights, gain, eps):
         rows in the compute type, the RMS norm of sum_t weights[t] X_t; else None. shift = (amount, state, batch): a row h
         becomes h + (h_before - h) * amount with h_before the request's row before, which `state` ([slots, width] 32-bit)
         keeps from step to step."""
@@ -1952,8 +1952,8 @@ class HipOps:
                 self._f32(bias, "mix_streams bias", D)
             self._f32(mix, "stream mix", S * S)
             self._f32(out, "stream factors", S)
-            # (a row before is worked out from the old streams again: they must stay)
-            new = x if x.dim() == 3 and shift is None else torch.empty(n, S, D, dtype=torch.float32, device=self.device)
+            # (the old streams are read again for a row before, and by the kernel for any sizes: they must stay)
+            new = torch.empty(n, S, D, dtype=torch.float32, device=self.device)
         h = weights = gain = amount = state = batch = None
         eps = 0.0
         if read is not None:
