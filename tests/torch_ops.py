@@ -71,6 +71,9 @@ class TorchOps:
             y = y + residual.float()
         return y.to(out_dtype or self.dtype)
 
+    def linear_act(self, x, w, act):
+        return self.activate_rows(self.linear(x, w, out_dtype=torch.float32), act)
+
     def linear_swiglu(self, x, w, rms=None):
         return self.swiglu(self.linear(x, w, rms=rms))
 

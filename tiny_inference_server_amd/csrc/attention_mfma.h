@@ -19,13 +19,14 @@ int tis_attention_mfma(const void* q, long q_ld, const void* plane, const int* b
                        int min_steps, int tile_splits, int tile_max_steps, int* row_splits, hipStream_t stream);
 
 // tis_attention_mfma with a sink in every row's softmax where sink != 0 (one more key without a value, of score 0 or, where
-// sinks is given, sinks[head]).
+// sinks is given, sinks[head]) and, where turn is given ([rows][head size / 2] pairs of (cos, sin)), every pair (2m, 2m + 1) of
+// a row's results turned back by that angle.
 int tis_attention_mfma_sink(const void* q, long q_ld, const void* plane, const int* block_tables, int bt_ld,
                             const int* row_seq, const int* positions, const int* items, int n_items, int nb,
                             const int* tiles, int n_tiles, void* out, long out_ld, float* part_o, float* part_ml, int rows,
                             int n_heads, int n_kv_heads, int head_dim, int page_size, int window, float scale, int n_splits,
                             int min_steps, int tile_splits, int tile_max_steps, int* row_splits, int sink,
-                            const float* sinks, hipStream_t stream);
+                            const float* sinks, const float* turn, hipStream_t stream);
 
 // A second stream (default priority, as `stream` must have) on which a call that holds both tiles and items runs its
 // tile kernel, beside the items' kernel on `stream`; the two meet again before the merge, and everything after the

@@ -83,6 +83,18 @@ __device__ __forceinline__ float sink_share(const float* sinks, int head, float 
   return __builtin_amdgcn_exp2f((sinks ? sinks[head] * 1.4426950408889634f : 0.f) - m);
 }
 
+// Values that were turned by their position before they were cached: a result's pairs (2m, 2m + 1) are turned back by the
+// row's angle, whose (cos, sin) is turn[m] of the row. Four consecutive channels of a lane; or one channel a lane, the
+// pair's other one on the neighbouring lane (head sizes are multiples of 16: both are there).
+__device__ __forceinline__ void turn_back(f32x4& v, const float2* turn) {
+  const float2 a = turn[0], b = turn[1];
+  v = (f32x4){v[0] * a.x + v[1] * a.y, v[1] * a.x - v[0] * a.y, v[2] * b.x + v[3] * b.y, v[3] * b.x - v[2] * b.y};
+}
+__device__ __forceinline__ float turn_back_lane(float v, int lane, float2 cs) {
+  const float other = __shfl_xor(v, 1, 64);
+  return lane & 1 ? v * cs.x - other * cs.y : v * cs.x + other * cs.y;
+}
+
 // PS16: pages of exactly 16 tokens. A 16-key tile is then a whole page, page indices are shifts, and a lane's
 // offsets inside a page never change: the loads of a step need no address arithmetic beyond the page's base.
 template <int NB, bool PS16>
@@ -91,7 +103,7 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(NB <= 2 ? 2 
     int bt_ld, const int* __restrict__ row_seq, const int* __restrict__ positions, const int2* __restrict__ items,
     bf16* __restrict__ out, long out_ld, float* __restrict__ part_o, float2* __restrict__ part_ml, int group_size,
     int n_kv_heads, int n_heads, int page_size_arg, int window, float scale_log2, int n_splits, int min_steps,
-    int split_stride, int* __restrict__ row_splits, int sink, const float* __restrict__ sinks) {
+    int split_stride, int* __restrict__ row_splits, int sink, const float* __restrict__ sinks, const float2* __restrict__ turn) {
   const int page_size = PS16 ? 16 : page_size_arg;
   const int item = blockIdx.x, kvh = blockIdx.y;
   int split = blockIdx.z;
@@ -368,7 +380,10 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(NB <= 2 ? 2 
       for (int db = 0; db < DB; ++db) {
         bf16x4 w;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) w[i] = static_cast<__bf16>(o[nb][db][i] * inv);
+        for (int i = 0; i < 4; ++i) o[nb][db][i] *= inv;
+        if (turn) turn_back(o[nb][db], turn + (long)col_row[nb] * (HD / 2) + (db * 16 + g * 4) / 2);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) w[i] = static_cast<__bf16>(o[nb][db][i]);
         *reinterpret_cast<bf16x4*>(dst + db * 16) = w;
       }
     } else {
@@ -448,7 +463,7 @@ __global__ __launch_bounds__(TW * 64) __attribute__((amdgpu_waves_per_eu(HD <= 1
     int bt_ld, const int* __restrict__ row_seq, const int* __restrict__ positions, const int2* __restrict__ tiles,
     bf16* __restrict__ out, long out_ld, float* __restrict__ part_o, float2* __restrict__ part_ml, int group_size,
     int n_kv_heads, int n_heads, int page_size_arg, int window, float scale_log2, int n_splits, int max_steps,
-    int split_stride, int* __restrict__ row_splits, int sink, const float* __restrict__ sinks) {
+    int split_stride, int* __restrict__ row_splits, int sink, const float* __restrict__ sinks, const float2* __restrict__ turn) {
   __shared__ __attribute__((aligned(16))) bf16 k_lds[TBUF][TCH * 8];
   __shared__ __attribute__((aligned(16))) bf16 v_lds[TBUF][TCH * 8];
   const int page_size = PS16 ? 16 : page_size_arg;
@@ -730,8 +745,12 @@ __global__ __launch_bounds__(TW * 64) __attribute__((amdgpu_waves_per_eu(HD <= 1
       for (int b = 0; b < 4; ++b) {
         if (HD % 32 != 0 && dt * 32 + b * 8 >= HD) continue;
         bf16x4 w;
+        f32x4 v;
 #pragma unroll
-        for (int k = 0; k < 4; ++k) w[k] = static_cast<__bf16>(o[dt][b * 4 + k] * inv);
+        for (int k = 0; k < 4; ++k) v[k] = o[dt][b * 4 + k] * inv;
+        if (turn) turn_back(v, turn + (long)col_row * (HD / 2) + (dt * 32 + b * 8 + h * 4) / 2);
+#pragma unroll
+        for (int k = 0; k < 4; ++k) w[k] = static_cast<__bf16>(v[k]);
         *reinterpret_cast<bf16x4*>(dst + dt * 32 + b * 8) = w;
       }
   } else {
@@ -758,7 +777,7 @@ __global__ __launch_bounds__(MG * 64) void attention_merge_kernel(const float* _
                                                                   const float2* __restrict__ part_ml,
                                                                   bf16* __restrict__ out, long out_ld, int n_heads,
                                                                   int max_splits, const int* __restrict__ row_splits,
-                                                                  int sink, const float* __restrict__ sinks) {
+                                                                  int sink, const float* __restrict__ sinks, const float2* __restrict__ turn) {
   __shared__ float so[MG][MD][64];
   const long row = blockIdx.x;
   const int head = blockIdx.y;
@@ -820,6 +839,7 @@ __global__ __launch_bounds__(MG * 64) void attention_merge_kernel(const float* _
     float t = so[0][j][lane];
 #pragma unroll
     for (int gq = 1; gq < MG; ++gq) t += so[gq][j][lane];
+    if (turn) t = turn_back_lane(t, lane, turn[row * (HD / 2) + d / 2]);
     out[row * out_ld + (long)head * HD + d] = static_cast<__bf16>(t / L);
   }
 }
@@ -832,7 +852,7 @@ __global__ __launch_bounds__(MG * 64) void attention_merge_rows_kernel(const flo
                                                                        const float2* __restrict__ part_ml,
                                                                        bf16* __restrict__ out, long out_ld,
                                                                        int n_heads, int max_splits,
-                                                                       const int* __restrict__ row_splits, int sink, const float* __restrict__ sinks) {
+                                                                       const int* __restrict__ row_splits, int sink, const float* __restrict__ sinks, const float2* __restrict__ turn) {
   const long row = blockIdx.x;
   const int n_splits = row_splits ? row_splits[row] : max_splits;
   if (n_splits <= 1) return;
@@ -873,7 +893,10 @@ __global__ __launch_bounds__(MG * 64) void attention_merge_rows_kernel(const flo
 #pragma unroll
   for (int j = 0; j < MD; ++j) {
     const int d = j * 64 + lane;
-    if (d < HD) out[row * out_ld + (long)head * HD + d] = static_cast<__bf16>(acc[j] / L);
+    if (d < HD) {
+      if (turn) acc[j] = turn_back_lane(acc[j], lane, turn[row * (HD / 2) + d / 2]);
+      out[row * out_ld + (long)head * HD + d] = static_cast<__bf16>(acc[j] / L);
+    }
   }
 }
 
@@ -934,7 +957,8 @@ static int attention_launch(const void* q, long q_ld, const void* plane, const i
                             const int* tiles, int n_tiles, void* out, long out_ld, float* part_o,
                             float* part_ml, int rows, int n_heads, int n_kv_heads, int head_dim, int page_size,
                             int window, float scale, int n_splits, int min_steps, int tile_splits,
-                            int tile_max_steps, int* row_splits, hipStream_t stream, int sink = 0, const float* sinks = nullptr) {
+                            int tile_max_steps, int* row_splits, hipStream_t stream, int sink = 0, const float* sinks = nullptr,
+                            const float2* turn = nullptr) {
   if ((n_items == 0 && n_tiles == 0) || rows == 0) return 0;
   if (n_items < 0 || n_tiles < 0 || (n_tiles > 0 && !tiles)) return tis_fail("attention_mfma: bad item counts %d, %d", n_items, n_tiles);
   if (head_dim != HD) return tis_fail("attention_mfma: built for head size %d, called with %d", HD, head_dim);
@@ -994,7 +1018,7 @@ static int attention_launch(const void* q, long q_ld, const void* plane, const i
   attention_mfma_kernel<NBV, PSV><<<grid, 64, 0, stream>>>(                                                      \
       (const bf16*)q, q_ld, (const bf16*)plane, block_tables, bt_ld, row_seq, positions, (const int2*)items,     \
       (bf16*)out, out_ld, part_o, (float2*)part_ml, group, n_kv_heads, n_heads, page_size, window, scale_log2,   \
-      n_splits, min_steps, stride, row_splits, sink, sinks)
+      n_splits, min_steps, stride, row_splits, sink, sinks, turn)
     if (page_size == 16) {
       if (nb == 1) LAUNCH(1, true);
       else if (nb == 2) LAUNCH(2, true);
@@ -1013,7 +1037,7 @@ static int attention_launch(const void* q, long q_ld, const void* plane, const i
   attention_tile_kernel<PSV><<<grid, TW * 64, 0, tile_stream>>>(                                                      \
       (const bf16*)q, q_ld, (const bf16*)plane, block_tables, bt_ld, row_seq, positions, (const int2*)tiles,     \
       (bf16*)out, out_ld, part_o, (float2*)part_ml, group, n_kv_heads, n_heads, page_size, window, scale_log2,   \
-      tile_splits, tile_max_steps, stride, row_splits, sink, sinks)
+      tile_splits, tile_max_steps, stride, row_splits, sink, sinks, turn)
     if (page_size == 16) LAUNCH(true);
     else LAUNCH(false);
 #undef LAUNCH
@@ -1027,11 +1051,11 @@ static int attention_launch(const void* q, long q_ld, const void* plane, const i
     if ((long)rows * n_heads > 8192) {
       dim3 mgrid(rows, (n_heads + MG - 1) / MG);
       attention_merge_rows_kernel<<<mgrid, MG * 64, 0, stream>>>(part_o, (const float2*)part_ml, (bf16*)out, out_ld,
-                                                                 n_heads, stride, row_splits, sink, sinks);
+                                                                 n_heads, stride, row_splits, sink, sinks, turn);
     } else {
       dim3 mgrid(rows, n_heads);
       attention_merge_kernel<<<mgrid, MG * 64, 0, stream>>>(part_o, (const float2*)part_ml, (bf16*)out, out_ld,
-                                                            n_heads, stride, row_splits, sink, sinks);
+                                                            n_heads, stride, row_splits, sink, sinks, turn);
     }
     rc = tis_launch_status("attention_merge");
   }
@@ -1051,16 +1075,17 @@ TIS_EXPORT int tis_attention_mfma(const void* q, long q_ld, const void* plane, c
 
 // The same with a sink in every row's softmax (sink != 0): the denominator also counts one key that has no value, of score
 // 0 or (sinks not null, one number per query head) sinks[head], which is not scaled; a row's weights add up to less than one.
+// turn (null: nothing): [rows][head size / 2] (cos, sin) by which the pairs (2m, 2m + 1) of a row's results are turned back.
 TIS_EXPORT int tis_attention_mfma_sink(const void* q, long q_ld, const void* plane, const int* block_tables, int bt_ld,
                                        const int* row_seq, const int* positions, const int* items, int n_items, int nb,
                                        const int* tiles, int n_tiles, void* out, long out_ld, float* part_o,
                                        float* part_ml, int rows, int n_heads, int n_kv_heads, int head_dim, int page_size,
                                        int window, float scale, int n_splits, int min_steps, int tile_splits,
                                        int tile_max_steps, int* row_splits, int sink, const float* sinks,
-                                       hipStream_t stream) {
+                                       const float* turn, hipStream_t stream) {
   return attention_launch(q, q_ld, plane, block_tables, bt_ld, row_seq, positions, items, n_items, nb, tiles, n_tiles,
                           out, out_ld, part_o, part_ml, rows, n_heads, n_kv_heads, head_dim, page_size, window, scale,
-                          n_splits, min_steps, tile_splits, tile_max_steps, row_splits, stream, sink, sinks);
+                          n_splits, min_steps, tile_splits, tile_max_steps, row_splits, stream, sink, sinks, (const float2*)turn);
 }
 
 // ---- the same without a workspace argument: partial results in memory that this library owns for good ----

@@ -37,7 +37,15 @@ typedef __attribute__((ext_vector_type(4))) __bf16 bf16x4;
 typedef __attribute__((ext_vector_type(4))) float f32x4;
 
 
-enum { EPI_NONE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ROPE = 3 };
+enum { EPI_NONE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ROPE = 3, EPI_GELU = 4, EPI_RELU2 = 5 };
+
+// what the epilogues EPI_GELU and EPI_RELU2 make of a 32-bit sum: the tanh form of gelu, 0.5 z (1 + tanh(u)) written as
+// z / (1 + exp(-2u)), and the square of relu
+template <int EPI> __device__ __forceinline__ float activated(float z) {
+  if (EPI == EPI_GELU) return z / (1.f + __expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
+  if (EPI == EPI_RELU2) { const float p = fmaxf(z, 0.f); return p * p; }
+  return z;
+}
 
 // What the rotary epilogue needs beyond the product: the rows of W are [q heads | k heads | v heads], and inside
 // every q and k head the rows are ordered so that the two members of a rotary pair are neighbours
@@ -74,7 +82,7 @@ __global__ __launch_bounds__(GS_WAVES * 64) void gemm_skinny_kernel(
     const bf16* __restrict__ X, long x_ld, const bf16* __restrict__ W, const float* __restrict__ gain, float eps,
     const bf16* __restrict__ R_in, long r_ld, TO* __restrict__ C, long c_ld, int M, int N, int K, RopeArgs rope) {
   static_assert(MB == 1 || R == 1, "several row blocks go with full column tiles only");
-  static_assert(CT == 1 || (R == 1 && (EPI == EPI_NONE || EPI == EPI_SWIGLU)), "two column tiles: plain and gated products");
+  static_assert(CT == 1 || (R == 1 && EPI != EPI_RESIDUAL && EPI != EPI_ROPE), "two column tiles: plain, gated and activated products");
   constexpr int COLS = 16 / R;   // output columns of a workgroup, and the most rows of X a block takes
   constexpr int GH = 4 / R;      // lane groups of four result rows per chunk
   __shared__ float red[GS_WAVES][MB][CT][64][4];
@@ -295,7 +303,7 @@ __global__ __launch_bounds__(GS_WAVES * 64) void gemm_skinny_kernel(
         if (n + i < N) {
           float t = v[i];
           if (EPI == EPI_RESIDUAL) t += res[mb][i];
-          C[(long)m * c_ld + n + i] = from_f<TO>(t);
+          C[(long)m * c_ld + n + i] = from_f<TO>(activated<EPI>(t));
         }
       }
     }
@@ -576,7 +584,7 @@ __global__ __launch_bounds__(512) void gemm_staged_kernel(
         if (n + i < N) {
           float s = v[i];
           if (EPI == EPI_RESIDUAL) s += res[j][i];
-          C[(long)m * c_ld + n + i] = from_f<TO>(s);
+          C[(long)m * c_ld + n + i] = from_f<TO>(activated<EPI>(s));
         }
       }
     }
@@ -607,7 +615,7 @@ static int launch_staged(const void* X, long x_ld, const void* W, const float* g
   // two column tiles a workgroup where that still leaves a workgroup for every compute unit: the panel's activations,
   // which a workgroup copies in full, then serve twice as many weights
   int ct = 1;
-  if constexpr (EPI == EPI_NONE || EPI == EPI_SWIGLU) {
+  if constexpr (EPI != EPI_RESIDUAL && EPI != EPI_ROPE) {
     if ((long)((N + 31) / 32) * panels >= g_wide_tiles) ct = 2;
   }
   const dim3 grid((N + 16 * ct - 1) / (16 * ct), panels);
@@ -623,7 +631,7 @@ static int launch_staged(const void* X, long x_ld, const void* W, const float* g
     return 0;                                                                                                     \
   }
   STAGED(2, 1, 4) STAGED(2, 1, 2) STAGED(1, 1, 4) STAGED(1, 1, 2)
-  if constexpr (EPI == EPI_NONE || EPI == EPI_SWIGLU) { STAGED(2, 2, 4) STAGED(2, 2, 2) STAGED(1, 2, 4) STAGED(1, 2, 2) }
+  if constexpr (EPI != EPI_RESIDUAL && EPI != EPI_ROPE) { STAGED(2, 2, 4) STAGED(2, 2, 2) STAGED(1, 2, 4) STAGED(1, 2, 2) }
 #undef STAGED
   return tis_fail("gemm_skinny: no staged kernel for %d column tiles and %d stages", ct, ns);
 }
@@ -669,7 +677,7 @@ static int launch_mb(const void* X, long x_ld, const void* W, const float* gain,
   return tis_launch_status("gemm_skinny");
 }
 
-// epilogue: 0 none, 1 residual, 2 swiglu. out_dtype: 0 float, 1 bfloat16. gain == null: no norm.
+// epilogue: 0 none, 1 residual, 2 swiglu, 4 tanh-form gelu, 5 the square of relu (both without a norm). out_dtype: 0 float, 1 bfloat16. gain == null: no norm.
 TIS_EXPORT int tis_gemm_skinny(const void* X, long x_ld, const void* W, const float* gain, float eps, const void* R,
                                long r_ld, void* C, long c_ld, int M, int N, int K, int epilogue, int out_dtype,
                                hipStream_t stream) {
@@ -686,6 +694,8 @@ TIS_EXPORT int tis_gemm_skinny(const void* X, long x_ld, const void* W, const fl
     if (epilogue == EPI_NONE) { if (norm) GO(true, EPI_NONE, bf16); else GO(false, EPI_NONE, bf16); }
     if (epilogue == EPI_RESIDUAL) { if (norm) GO(true, EPI_RESIDUAL, bf16); else GO(false, EPI_RESIDUAL, bf16); }
     if (epilogue == EPI_SWIGLU) { if (norm) GO(true, EPI_SWIGLU, bf16); else GO(false, EPI_SWIGLU, bf16); }
+    if (epilogue == EPI_GELU && !norm) GO(false, EPI_GELU, bf16);
+    if (epilogue == EPI_RELU2 && !norm) GO(false, EPI_RELU2, bf16);
   } else if (out_dtype == TIS_F32) {
     if (epilogue == EPI_NONE) { if (norm) GO(true, EPI_NONE, float); else GO(false, EPI_NONE, float); }
   }

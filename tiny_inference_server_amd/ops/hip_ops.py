@@ -89,7 +89,7 @@ _SIGNATURES["gemm_skinny"] = ("tis_gemm_skinny", {
     "tis_gemm_skinny_qkv_rope": [_P, _L, _P, _P, _F, _P, _L, _I, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
 })
 _SIGNATURES["gemm_tiles"] = ("tis_gemm_tiles", {
-    "tis_gemm_tiles": [_P, _L, _P, _P, _L, _P, _L, _I, _I, _I, _I, _P],
+    "tis_gemm_tiles": [_P, _L, _P, _P, _L, _P, _L, _I, _I, _I, _I, _I, _P],
 })
 _SIGNATURES["gemm_library"] = ("tis_gemm_library", {
     "tis_gemm_library_init": [],
@@ -100,7 +100,7 @@ _SIGNATURES["attention_mfma"] = ("tis_attention_mfma", {
     "tis_attention_mfma": [_P, _L, _P, _P, _I, _P, _P, _P, _I, _I, _P, _I, _P, _L, _P, _P, _I, _I, _I, _I, _I, _I, _F,
                            _I, _I, _I, _I, _P, _P],
     "tis_attention_mfma_sink": [_P, _L, _P, _P, _I, _P, _P, _P, _I, _I, _P, _I, _P, _L, _P, _P, _I, _I, _I, _I, _I, _I, _F,
-                                _I, _I, _I, _I, _P, _I, _P, _P],
+                                _I, _I, _I, _I, _P, _I, _P, _P, _P],
 })
 
 _SIGNATURES["stream32"] = ("tis_stream32", {
@@ -165,8 +165,7 @@ _SIGNATURES["hyper_streams"] = ("tis_hyper_streams", {
 })
 _SIGNATURES["convolved_attention"] = ("tis_convolved", {
     "tis_convolved_prepare": [_I, _P, _L, _P, _P, _P, _L, _P, _P, _P, _P, _P, _P, _P, _L, _P, _I, _F, _P, _P, _I, _I, _I, _I, _I, _I,
-                              _I, _I, _P],
-    "tis_turn_back": [_I, _P, _L, _P, _I, _I, _I, _P],
+                              _I, _P],
 })
 
 _libs = {}
@@ -837,7 +836,7 @@ class HipOps:
             out = self.empty(M, N, dtype=out_dtype)
             self.gemm_tiles.tis_gemm_tiles(_ptr(x), x.stride(0), _ptr(w), _ptr(residual),
                                            residual.stride(0) if residual is not None else 0, _ptr(out), out.stride(0),
-                                           M, N, K, 1 if out_dtype == torch.float32 else 0, self._stream())
+                                           M, N, K, 1 if out_dtype == torch.float32 else 0, 0, self._stream())
             return out
         out = self.empty(M, N, dtype=out_dtype)
         self.gemm_plain.tis_gemm_plain(1, _DT[out_dtype], _ptr(x), x.stride(0), _ptr(w), K, _ptr(residual),
@@ -882,6 +881,31 @@ class HipOps:
                 _ptr(None), 0, _ptr(out), out.stride(0), M, N, K, 2, 1, self._stream())
             return out
         return self.swiglu(self.linear(x, w, rms=rms))
+
+    # activations that a bfloat16 product applies to its 32-bit sums: (few-row kernel's epilogue, tiled kernel's code)
+    _PRODUCT_ACTS = {"gelu_tanh": (4, 1), "relu2": (5, 2)}
+
+    def linear_act(self, x, w, act: str):
+        """act(x . w^T) in the compute type, the activation taken on the 32-bit sums: [M, N]. act: "gelu_tanh", "relu2" (the
+        square of relu), or another of activate_rows, which then runs after the product."""
+        _rows_view(self._check(x, "linear x"), "linear x")
+        self._check(w, "linear w")
+        M, K = x.shape
+        if w.dim() != 2 or w.shape[1] != K or not w.is_contiguous():
+            raise KernelError(f"linear: x {tuple(x.shape)} against w {tuple(w.shape)} (w is [out, in], contiguous)")
+        N = w.shape[0]
+        codes = self._PRODUCT_ACTS.get(act)
+        route = self._route(x, M, N, K, torch.float32) if self.dtype == torch.bfloat16 and M else "plain"
+        if codes is None or route not in ("few_rows", "tiles"):
+            return self.activate_rows(self.linear(x, w, out_dtype=torch.float32), act)
+        out = self.empty(M, N)
+        if route == "few_rows":
+            self.gemm_skinny.tis_gemm_skinny(_ptr(x), x.stride(0), _ptr(w), _ptr(None), 0.0, _ptr(None), 0, _ptr(out), out.stride(0),
+                                             M, N, K, codes[0], 1, self._stream())
+        else:
+            self.gemm_tiles.tis_gemm_tiles(_ptr(x), x.stride(0), _ptr(w), _ptr(None), 0, _ptr(out), out.stride(0), M, N, K, 0,
+                                           codes[1], self._stream())
+        return out
 
     @staticmethod
     def _holds_rows(t, rows: int) -> bool:
@@ -1012,6 +1036,8 @@ class HipOps:
         """
         group_name = group
         sink, sinks = self._sink(sink, n_heads)
+        if turn is not None:
+            self._turn(turn, q.shape[0], head_dim)
         if (sink or gate is not None or turn is not None) and slopes is not None:
             raise KernelError("attention: score slopes go with neither a sink nor a gate nor turned values")
         _rows_view(self._check(q, "q"), "q")
@@ -1116,9 +1142,7 @@ class HipOps:
                                         n_tiles, _ptr(out), out.stride(0), _ptr(part_o), _ptr(part_ml), n, n_heads,
                                         n_kv_heads, head_dim, page_size, int(window), float(scale), n_splits, min_steps,
                                         tile_splits, tile_max_steps, _ptr(row_splits), 1 if sink else 0, _ptr(sinks),
-                                        self._stream())
-            if turn is not None:
-                self.turn_back(out, turn, n_heads, head_dim)
+                                        _ptr(turn), self._stream())
             if gate is not None:
                 self.head_gate(out, gate, n_heads, head_dim)
             return out
@@ -1145,17 +1169,6 @@ class HipOps:
         if dim % 2:
             raise KernelError(f"attention: values of {dim} channels cannot be turned back in pairs")
         return self._f32(turn, "angles of turned values", n * dim)
-
-    def turn_back(self, x, turn, n_heads: int, dim: int):
-        """In place: the pairs (2m, 2m + 1) of every head of x [rows, heads * dim] (compute type) are turned back by the
-        angle whose (cos, sin) is turn[row, m]; turn: [rows, dim / 2, 2] 32-bit."""
-        _rows_view(self._check(x, "turn_back x"), "turn_back x")
-        n = x.shape[0]
-        if x.shape[1] != n_heads * dim:
-            raise KernelError(f"turn_back: x {tuple(x.shape)} for {n_heads} heads of {dim}")
-        self._turn(turn, n, dim)
-        self._lazy("convolved_attention").tis_turn_back(self.code, _ptr(x), x.stride(0), _ptr(turn), n, n_heads, dim, self._stream())
-        return x
 
     # ---- a residual stream in 32-bit, norm after the sum ------------------------------------------------
     # The libraries below are loaded when a model first asks for them: a model that has no such part never
@@ -1916,14 +1929,12 @@ class HipOps:
         self._check_kv_plane(plane, n_kv_heads, key_dim, value_dim, page_size)
         q = self.empty(n, n_heads * key_dim)
         turn = torch.empty(n, value_dim // 2, 2, dtype=torch.float32, device=self.device) if turn_freqs is not None else None
-        # rows a wave takes one after the other: with few rows one, so that a step still fills the chip
-        chunk = 1 if n <= 256 else 8
         self._lazy("convolved_attention").tis_convolved_prepare(
             self.code, _ptr(proj), proj.stride(0), _ptr(bias), _ptr(taps), _ptr(state if K > 1 else None),
             state.stride(0) if K > 1 else 0, _ptr(batch.row_seq), _ptr(batch.cu_rows), _ptr(batch.seq_slots),
             _ptr(batch.positions), _ptr(write_slots), _ptr(plane), _ptr(q), q.stride(0), _ptr(freqs if rot_dims else None),
             int(rot_dims), float(rot_factor), _ptr(turn_freqs), _ptr(turn), n, K, n_heads, n_kv_heads, key_dim, value_dim,
-            page_size, chunk, self._stream())
+            page_size, self._stream())
         return q, turn
 
     # ---- a residual of several streams -------------------------------------------------------------------------------

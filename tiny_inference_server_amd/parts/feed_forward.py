@@ -208,8 +208,7 @@ class ActivatedDense:
 
     def forward32(self, rows):
         ops = self.ops
-        hidden = ops.activate_rows(ops.linear(rows, self.w_up, out_dtype=torch.float32), self.act)
-        return ops.linear(hidden, self.w_down, out_dtype=torch.float32)
+        return ops.linear(ops.linear_act(rows, self.w_up, self.act), self.w_down, out_dtype=torch.float32)
 
     def forward(self, x, residual=None):
         y = self.forward32(x)
