@@ -3,17 +3,15 @@
 // Built once per (KD, VD): -DTIS_LATENT=KD*10000+VD.
 //
 // Pages of 16 slots hold the keys as [slot][KD] and then the values transposed, [VD][slot] (the layout of every
-// attention kernel of this engine with one key/value head). One wave takes an item: 16 columns that share their keys,
-// a column being a (row, query head) pair: with 16 heads or more a row's heads in blocks of 16, with fewer heads as many
-// consecutive rows of one request as fit. Keys go by in steps of 32 (two pages):
-//   S^T = K . Q^T    keys are the A operand straight from memory (16 bytes a lane), the queries stay in registers
-//   O^T += V^T . P^T the transposed values are the A operand straight from memory, the weights never leave registers
-// both on v_mfma_f32_16x16x32_bf16. The lane that holds a column's scores of the keys 4g .. 4g+3 of both pages feeds
-// exactly those eight as its share of P^T, and takes the values of the same eight keys: the contraction's order is
-// free as long as both operands agree. Softmax in 32-bit with a running maximum per column. Slots behind a row's
+// attention kernel of this engine with one key/value head). 16 columns share their keys, a column being a (row, query head)
+// pair. Keys go by in pages:
+//   S^T = K . Q^T    keys and queries are the operands of v_mfma_f32_16x16x32_bf16
+//   O^T += V^T . P^T the transposed values and the weights, rounded to bfloat16, likewise
+// The contraction's order is free as long as both operands agree, so a lane that holds a column's scores of four keys of a
+// page feeds exactly those as its share of P^T. Softmax in 32-bit with a running maximum per column. Slots behind a row's
 // position are read (their page is mapped) but their scores become -inf and their values zero before any arithmetic.
 // A long key range is cut into `n_splits` parts (grid z) whose partial results a second kernel merges. window > 0: a row
-// sees its last `window` keys only; steps that no row of an item sees are left out, and slots before the first key any
+// sees its last `window` keys only; pages that no row of an item sees are left out, and slots before the first key any
 // row sees (their page may have gone to another request) are treated like those behind the last. sinks (nullable): head h's
 // softmax has one more key of score sinks[h], not scaled, without a value.
 #include "common.h"
@@ -46,123 +44,152 @@ __device__ __forceinline__ float quad_sum(float v) {
   return v + __shfl_xor(v, 32, 64);
 }
 
-__global__ __launch_bounds__(64) void latent_mfma_kernel(
+// Single rows: a workgroup of four waves takes a row's heads in blocks of 16 and one part of its keys, four pages at a time.
+// Wave w multiplies page w's keys with the queries (from LDS, where they lie once for all four); the columns' maxima and the
+// weights, rounded to bfloat16, meet in LDS; then every wave adds up all 64 keys for its share of the value channels (every
+// fourth block of 16). So a workgroup has everything it needs of four pages on its way at once, in four short chains.
+static constexpr int DEC_PAGES = 4, DEC_KEYS = DEC_PAGES * PAGE;
+static constexpr int DEC_DB = (DB + 3) / 4;                    // blocks of value channels a wave takes
+static constexpr int DQ_STRIDE = KD + 8;                       // elements between two columns' queries in LDS
+
+__global__ __launch_bounds__(256) void latent_decode_kernel(
     const bf16* __restrict__ q, long ldq, const bf16* __restrict__ plane, const int* __restrict__ block_tables, int bt_ld,
-    const int* __restrict__ row_seq, const int* __restrict__ positions, const int2* __restrict__ items,
-    bf16* __restrict__ out, long ldo, float* __restrict__ part_o, float2* __restrict__ part_ml, int H, float scale_log2,
-    int n_splits, int window, const float* __restrict__ sinks) {
-  const int item = blockIdx.x, hb = blockIdx.y, split = blockIdx.z;
-  const int lane = threadIdx.x, c16 = lane & 15, g = lane >> 4;
-  const int row0 = items ? items[item].x : item;
-  const int n_rows = items ? items[item].y : 1;
-  const int p_first = positions[row0];
-  const int* bt = block_tables + (long)row_seq[row0] * bt_ld;
-  const int p_last = p_first + n_rows - 1;
-  // the lane's column
-  const int ro = H >= 16 ? 0 : c16 / H;
-  const int head = H >= 16 ? hb * 16 + c16 : c16 % H;
-  const bool col_ok = ro < n_rows && head < H;
-  const int col_row = row0 + (col_ok ? ro : 0);
-  const int col_pos = col_ok ? p_first + ro : -1;
-  const int col_lo = window > 0 ? col_pos - window + 1 : 0;                // the column's first key
-  const int k_lo = window > 0 ? max(0, p_first - window + 1) : 0;          // the first key any column sees
+    const int* __restrict__ row_seq, const int* __restrict__ positions, bf16* __restrict__ out, long ldo,
+    float* __restrict__ part_o, float2* __restrict__ part_ml, int H, float scale_log2, int n_splits, int window,
+    const float* __restrict__ sinks) {
+  __shared__ __attribute__((aligned(16))) bf16 q_lds[16 * DQ_STRIDE];
+  __shared__ bf16x4 p_lds[DEC_PAGES][64];
+  __shared__ float col_lds[DEC_PAGES][16];
+  const long row = blockIdx.x;
+  const int hb = blockIdx.y, split = blockIdx.z;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), c16 = lane & 15, g = lane >> 4;
+  const int pos = positions[row];
+  const int* bt = block_tables + (long)row_seq[row] * bt_ld;
+  const int head = hb * 16 + c16;
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
-
-  bf16x8 qb[DC];
-#pragma unroll
-  for (int dc = 0; dc < DC; ++dc) {
-    const int d = dc * 32 + g * 8;
-    qb[dc] = (col_ok && d < KD) ? *reinterpret_cast<const bf16x8*>(q + (long)col_row * ldq + (long)head * KD + d) : zero8;
-  }
-
-  const int s_first = k_lo / 32, n_steps = p_last / 32 + 1 - s_first;
-  const int per = (n_steps + n_splits - 1) / n_splits;
-  const int s_begin = s_first + split * per, s_end = min(s_first + n_steps, s_begin + per);
-  f32x4 o[DB];
-#pragma unroll
-  for (int db = 0; db < DB; ++db) o[db] = (f32x4){0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
+  const int k_lo = window > 0 ? max(0, pos - window + 1) : 0;       // the first key the row sees
+  const int c_first = k_lo / DEC_KEYS, n_chunks = pos / DEC_KEYS + 1 - c_first;
+  const int per = (n_chunks + n_splits - 1) / n_splits;
+  const int c_begin = c_first + split * per, c_end = min(c_first + n_chunks, c_begin + per);
   const long page_stride = (long)PAGE * (KD + VD);
+  const int last_page = pos / PAGE, first_page = k_lo / PAGE;
 
-  for (int s = s_begin; s < s_end; ++s) {
-    const int kb = s * 32;
-    const bool ok1 = kb + 16 <= p_last;                       // the step's second page holds keys some row sees
-    const bf16* pg0 = plane + (long)bt[kb >> 4] * page_stride;
-    const bf16* pg1 = plane + (long)(ok1 ? bt[(kb >> 4) + 1] : bt[kb >> 4]) * page_stride;
+  for (int i = tid; i < 16 * (KD / 8); i += 256) {
+    const int col = i / (KD / 8), piece = i % (KD / 8);
+    *reinterpret_cast<bf16x8*>(q_lds + col * DQ_STRIDE + piece * 8) =
+        hb * 16 + col < H ? *reinterpret_cast<const bf16x8*>(q + row * ldq + (long)(hb * 16 + col) * KD + piece * 8) : zero8;
+  }
+  f32x4 o[DEC_DB];
+#pragma unroll
+  for (int i = 0; i < DEC_DB; ++i) o[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+  for (int chunk = c_begin; chunk < c_end; ++chunk) {
+    const int kb = chunk * DEC_KEYS;
+    // (a page that holds no key the row sees may belong to nobody: one that does is read in its place, and masked)
+    const bf16* pg[DEC_PAGES];
+#pragma unroll
+    for (int j = 0; j < DEC_PAGES; ++j) pg[j] = plane + (long)bt[min(max(chunk * DEC_PAGES + j, first_page), last_page)] * page_stride;
+    const bf16* mine = plane + (long)bt[min(max(chunk * DEC_PAGES + wave, first_page), last_page)] * page_stride;
+    bf16x8 k[DC];
+#pragma unroll
+    for (int dc = 0; dc < DC; ++dc) {
+      const int d = dc * 32 + g * 8;
+      k[dc] = d < KD ? *reinterpret_cast<const bf16x8*>(mine + (long)c16 * KD + d) : zero8;
+    }
+    bf16x4 v[DEC_DB][DEC_PAGES];
+#pragma unroll
+    for (int i = 0; i < DEC_DB; ++i) {
+      const int db = min(wave + 4 * i, DB - 1);
+#pragma unroll
+      for (int j = 0; j < DEC_PAGES; ++j)
+        v[i][j] = *reinterpret_cast<const bf16x4*>(pg[j] + (long)PAGE * KD + (long)(db * 16 + c16) * PAGE + 4 * g);
+    }
+    if (chunk == c_begin) __syncthreads();                          // the queries are there
     f32x4 st0 = {0.f, 0.f, 0.f, 0.f}, st1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int dc = 0; dc < DC; ++dc) {
       const int d = dc * 32 + g * 8;
-      const bf16x8 k0 = d < KD ? *reinterpret_cast<const bf16x8*>(pg0 + (long)c16 * KD + d) : zero8;
-      const bf16x8 k1 = (d < KD && ok1) ? *reinterpret_cast<const bf16x8*>(pg1 + (long)c16 * KD + d) : zero8;
-      st0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, qb[dc], st0, 0, 0, 0);
-      st1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, qb[dc], st1, 0, 0, 0);
+      const bf16x8 qv = d < KD ? *reinterpret_cast<const bf16x8*>(q_lds + c16 * DQ_STRIDE + d) : zero8;
+      if (dc & 1) st1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k[dc], qv, st1, 0, 0, 0);
+      else st0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k[dc], qv, st0, 0, 0, 0);
     }
-    // the lane holds, for its column, the scores of the keys kb + 4g + i (first page) and kb + 16 + 4g + i (second)
-    float sv[8];
-    float tmax = -INFINITY;
+    // the lane holds, for its column, the scores of the keys kb + 16 wave + 4g + i
+    float sv[4], tmax = -INFINITY;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int key0 = kb + 4 * g + i, key1 = key0 + 16;
-      sv[i] = (key0 <= col_pos && key0 >= col_lo) ? st0[i] * scale_log2 : -INFINITY;
-      sv[4 + i] = (ok1 && key1 <= col_pos && key1 >= col_lo) ? st1[i] * scale_log2 : -INFINITY;
-      tmax = fmaxf(tmax, fmaxf(sv[i], sv[4 + i]));
+      const int key = kb + wave * PAGE + 4 * g + i;
+      sv[i] = (key <= pos && key >= k_lo) ? (st0[i] + st1[i]) * scale_log2 : -INFINITY;
+      tmax = fmaxf(tmax, sv[i]);
     }
     tmax = quad_max(tmax);
-    const float m_new = fmaxf(m, tmax);
-    const float m_use = m_new == -INFINITY ? 0.f : m_new;     // a column with no key yet: everything stays 0
+    if (g == 0) col_lds[wave][c16] = tmax;
+    __syncthreads();
+    const float m_new = fmaxf(fmaxf(fmaxf(col_lds[0][c16], col_lds[1][c16]), fmaxf(col_lds[2][c16], col_lds[3][c16])), m);
+    const float m_use = m_new == -INFINITY ? 0.f : m_new;           // no key yet: everything stays 0
     const float alpha = exp2f(m - m_use);
+    bf16x4 p;
     float psum = 0.f;
-    bf16x8 pb;
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const float p = exp2f(sv[e] - m_use);
-      psum += p;
-      pb[e] = static_cast<__bf16>(p);
+    for (int i = 0; i < 4; ++i) {
+      const float w = exp2f(sv[i] - m_use);
+      psum += w;
+      p[i] = static_cast<__bf16>(w);
     }
+    p_lds[wave][lane] = p;
     l = l * alpha + psum;
     m = m_new;
-    const bool edge = kb + 31 > p_last || kb < k_lo;           // some of the step's slots lie behind or before what any row sees
+    __syncthreads();
+    const bool edge = kb + DEC_KEYS - 1 > pos || kb < k_lo;          // some of the slots lie outside what the row sees
+    bf16x8 pb[2];
 #pragma unroll
-    for (int db = 0; db < DB; ++db) {
-      const long off = (long)PAGE * KD + (long)(db * 16 + c16) * PAGE + 4 * g;
-      const bf16x4 lo = *reinterpret_cast<const bf16x4*>(pg0 + off);
-      const bf16x4 hi = ok1 ? *reinterpret_cast<const bf16x4*>(pg1 + off) : (bf16x4){0, 0, 0, 0};
-      bf16x8 va = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
-      if (edge) {
+    for (int t = 0; t < 2; ++t) {
+      const bf16x4 lo = p_lds[2 * t][lane], hi = p_lds[2 * t + 1][lane];
+      pb[t] = (bf16x8){lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+    }
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int key0 = kb + 4 * g + i, key1 = key0 + 16;
-          if (key0 > p_last || key0 < k_lo) va[i] = static_cast<__bf16>(0.f);
-          if (key1 > p_last || key1 < k_lo) va[4 + i] = static_cast<__bf16>(0.f);
+    for (int i = 0; i < DEC_DB; ++i) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) o[i][e] *= alpha;
+#pragma unroll
+      for (int t = 0; t < 2; ++t) {
+        const bf16x4 lo = v[i][2 * t], hi = v[i][2 * t + 1];
+        bf16x8 va = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+        if (edge) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const int key0 = kb + 2 * t * PAGE + 4 * g + e, key1 = key0 + PAGE;
+            if (key0 > pos || key0 < k_lo) va[e] = static_cast<__bf16>(0.f);
+            if (key1 > pos || key1 < k_lo) va[4 + e] = static_cast<__bf16>(0.f);
+          }
         }
+        o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va, pb[t], o[i], 0, 0, 0);
       }
-#pragma unroll
-      for (int i = 0; i < 4; ++i) o[db][i] *= alpha;
-      o[db] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va, pb, o[db], 0, 0, 0);
     }
   }
-
-  // the lane holds, for its column, the channels db * 16 + 4g + i
-  const float lt = quad_sum(l);
-  if (!col_ok) return;
-  if (n_splits == 1) {
-    const float inv = 1.f / (lt + sink_share(sinks, head, m));
-    bf16* dst = out + (long)col_row * ldo + (long)head * VD + 4 * g;
+  // (a split without chunks leaves a maximum of -inf, a sum and results of zero)
+  l = quad_sum(l);
+  __syncthreads();
+  if (g == 0) col_lds[wave][c16] = l;
+  __syncthreads();
+  const float lt = (col_lds[0][c16] + col_lds[1][c16]) + (col_lds[2][c16] + col_lds[3][c16]);
+  if (head >= H) return;
+  // the lane holds, for its column, the channels db * 16 + 4g + e of its wave's blocks
+  const long slot = (row * H + head) * n_splits + split;
+  const float inv = n_splits == 1 ? 1.f / (lt + sink_share(sinks, head, m)) : 1.f;
 #pragma unroll
-    for (int db = 0; db < DB; ++db) {
+  for (int i = 0; i < DEC_DB; ++i) {
+    const int db = wave + 4 * i;
+    if (db >= DB) continue;
+    if (n_splits == 1) {
       bf16x4 w;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) w[i] = static_cast<__bf16>(o[db][i] * inv);
-      *reinterpret_cast<bf16x4*>(dst + db * 16) = w;
+      for (int e = 0; e < 4; ++e) w[e] = static_cast<__bf16>(o[i][e] * inv);
+      *reinterpret_cast<bf16x4*>(out + row * ldo + (long)head * VD + db * 16 + 4 * g) = w;
+    } else {
+      *reinterpret_cast<f32x4*>(part_o + slot * VD + db * 16 + 4 * g) = o[i];
     }
-  } else {
-    const long slot = ((long)col_row * H + head) * n_splits + split;
-    float* dst = part_o + slot * VD + 4 * g;
-#pragma unroll
-    for (int db = 0; db < DB; ++db) *reinterpret_cast<f32x4*>(dst + db * 16) = o[db];
-    if (g == 0) part_ml[slot] = make_float2(m, lt);
   }
+  if (n_splits > 1 && g == 0 && wave == 0) part_ml[slot] = make_float2(m, lt);
 }
 
 // Portions of prompts: a workgroup of four waves takes an item of 64 columns (with fewer than 64 heads, 64 / heads
@@ -363,10 +390,9 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restri
 
 TIS_EXPORT int tis_attention_latent_dims() { return TIS_LATENT; }
 
-// items: (first row, rows) per item, or null where every item is the single row of its own index. part_o / part_ml:
-// [rows][H][n_splits][VD] floats and [rows][H][n_splits] (maximum, sum) pairs, needed where n_splits > 1.
-// n_splits 0: the items are those of the four-wave kernel (64 columns each: 64 / H rows, or a row's heads in blocks of
-// 64), which takes every item's keys whole.
+// items: (first row, rows) per item of the kernel for portions (64 columns each: 64 / H rows, or a row's heads in blocks of
+// 64), which takes every item's keys whole (n_splits 0). Null: `rows` single rows, whose keys are cut into n_splits parts;
+// part_o / part_ml: [rows][H][n_splits][VD] floats and [rows][H][n_splits] (maximum, sum) pairs where n_splits > 1.
 TIS_EXPORT int tis_attention_latent(const void* q, long ldq, const void* plane, const int* block_tables, int bt_ld,
                                     const int* row_seq, const int* positions, const int* items, int n_items, void* out,
                                     long ldo, float* part_o, float* part_ml, int rows, int H, int key_dim, int value_dim,
@@ -387,10 +413,11 @@ TIS_EXPORT int tis_attention_latent(const void* q, long ldq, const void* plane, 
                                                   scale * 1.4426950408889634f, window, sinks);
     return tis_launch_status("attention_latent tiles");
   }
-  dim3 grid(n_items, (H + 15) / 16, n_splits);
-  latent_mfma_kernel<<<grid, 64, 0, stream>>>((const bf16*)q, ldq, (const bf16*)plane, block_tables, bt_ld, row_seq, positions,
-                                             (const int2*)items, (bf16*)out, ldo, part_o, (float2*)part_ml, H,
-                                             scale * 1.4426950408889634f, n_splits, window, sinks);
+  if (items || n_items != rows) return tis_fail("attention_latent: single rows come without a list (%d items of %d rows)", n_items, rows);
+  dim3 grid(rows, (H + 15) / 16, n_splits);
+  latent_decode_kernel<<<grid, 256, 0, stream>>>((const bf16*)q, ldq, (const bf16*)plane, block_tables, bt_ld, row_seq, positions,
+                                                (bf16*)out, ldo, part_o, (float2*)part_ml, H, scale * 1.4426950408889634f,
+                                                n_splits, window, sinks);
   int rc = tis_launch_status("attention_latent");
   if (rc || n_splits == 1) return rc;
   dim3 mgrid(rows, H);

@@ -1843,14 +1843,12 @@ class HipOps:
             items, n_items = plan[0].reshape(-1), plan[1]
             if items.numel() < 2 * n_items or items.dtype != torch.int32 or not items.is_contiguous():
                 raise KernelError(f"attention: a list of {items.numel()} integers for {n_items} items")
-        # Portions: the four-wave kernel, every item's keys whole. Single rows: a wave per row and 16 heads, with
-        # enough waves to fill the chip: a request's keys are cut where its rows alone would leave most units idle
-        waves = n_items * -(-n_heads // 16)
-        steps = -(-(min(batch.max_kv_len, window + 31) if window else batch.max_kv_len) // 32)
+        # Portions: the kernel for items of 64 columns, every item's keys whole. Single rows: a workgroup per row, 16 heads
+        # and part of the keys, which it takes 64 at a time; a request's keys are cut into as many parts as fill the chip
+        # twice over (many short chains beat few long ones)
+        chunks = -(-(min(batch.max_kv_len, window + 63) if window else batch.max_kv_len) // 64)
         most = max(1, (self._workspace.numel() // (n * n_heads * (value_dim + 2))))
-        # (a wave's step is two or three dependent trips to memory and little else, so many short chains beat few long
-        # ones: four waves a compute unit, down to one step each)
-        n_splits = 0 if items is not None else int(max(1, min(-(-4 * self.units // waves), steps, 64, most)))
+        n_splits = 0 if items is not None else int(max(1, min(-(-2 * self.units // (n * -(-n_heads // 16))), chunks, 64, most)))
         part_o = part_ml = None
         if n_splits > 1:
             part_o = self._workspace
