@@ -339,6 +339,210 @@ __global__ __launch_bounds__(256) void latent_tile_kernel(
   }
 }
 
+// The same items on eight waves, where two buffers of a step's keys and values fit into LDS. What bounds an item is what its
+// workgroup reads from LDS, so the two products are cut differently: in the first a wave takes 16 columns and one of the
+// step's two pages (keys are read once per 16 columns), in the second all 64 columns and every eighth block of 16 value
+// channels (values are read once per workgroup; the weights, a sixteenth of their size, eight times). Keys and values go from
+// the pages straight into LDS (no registers) a step ahead. Key rows lie an odd number of 16-byte pieces apart and a value
+// channel's two pieces change places with every eighth channel, so that what sixteen lanes read at a time meets no bank
+// conflict. A column's running maximum is raised only when a step exceeds it by 2^8 (weights then stay below 2^8), and
+// sums are rescaled only in such steps. Sums run over the keys in order; a row's result does not depend on the item it is in.
+static constexpr int T8_KPS = (KD / 8) | 1;                           // 16-byte pieces from one key to the next in LDS
+static constexpr int T8_KI = (32 * T8_KPS + 63) / 64;                 // copies (64 pieces each) that bring a step's keys
+static constexpr int T8_VI = (4 * VD + 63) / 64;                      // ... and its values
+static constexpr int T8_LPW = (T8_KI + T8_VI + 7) / 8;                // copies a wave issues
+static constexpr int T8_V_AT = T8_KI * 1024, T8_STAGE = T8_V_AT + T8_VI * 1024;      // bytes
+static constexpr int T8_P_STRIDE = 80;                                // bytes from one column's weights to the next
+static constexpr int T8_P_AT = 2 * T8_STAGE, T8_BYTES = T8_P_AT + 64 * T8_P_STRIDE + (2 + 1 + 2) * 64 * 4;
+static constexpr bool T8_FITS = T8_BYTES <= 160 * 1024;
+static constexpr int T8_DB = (DB + 7) / 8;                            // blocks of value channels a wave takes
+
+#pragma clang diagnostic ignored "-Winline-asm"   // M0 in a clobber list: meant
+// One 16-byte piece per lane from global memory straight into LDS, lane i's at lds_addr + 16 i; whoever reads the pieces
+// waits for them (vmcnt) and for the other waves (barrier).
+__device__ __forceinline__ void lt_copy16(const void* lane_src, unsigned lds_addr) {
+  const unsigned base = (unsigned)__builtin_amdgcn_readfirstlane((int)lds_addr);
+  asm volatile("s_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, off" : : "v"(lane_src), "s"(base) : "memory", "m0");
+}
+
+template <bool FITS>
+__global__ __launch_bounds__(512) void latent_tile8_kernel(
+    const bf16* __restrict__ q, long ldq, const bf16* __restrict__ plane, const int* __restrict__ block_tables, int bt_ld,
+    const int* __restrict__ row_seq, const int* __restrict__ positions, const int2* __restrict__ items,
+    bf16* __restrict__ out, long ldo, int H, float scale_log2, int window, const float* __restrict__ sinks) {
+  __shared__ __attribute__((aligned(1024))) unsigned char lds[FITS ? T8_BYTES : 16];
+  if (!FITS) return;
+  const unsigned lds0 = (unsigned)(uintptr_t)(const __attribute__((address_space(3))) unsigned char*)lds;
+  unsigned char* p_lds = lds + T8_P_AT;                               // [64 columns][32 keys] bfloat16
+  float* max_lds = reinterpret_cast<float*>(p_lds + 64 * T8_P_STRIDE);      // [2 pages][64]: a step's maxima
+  float* alpha_lds = max_lds + 128;                                   // [64]: what a column's sums are rescaled by
+  float* sum_lds = alpha_lds + 64;                                    // [2][64]
+  const int item = blockIdx.x, hb = blockIdx.y;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), c16 = lane & 15, g = lane >> 4;
+  const int ct = wave & 3, kt = wave >> 2;                            // first product: the wave's 16 columns, its page
+  const int row0 = items[item].x, n_rows = items[item].y;
+  const int p_first = positions[row0], p_last = p_first + n_rows - 1;
+  const int* bt = block_tables + (long)row_seq[row0] * bt_ld;
+  // column c of the item: its row, its head, whether there is one
+  auto row_of = [&](int c) { return H >= 64 ? 0 : c / H; };
+  auto head_of = [&](int c) { return H >= 64 ? hb * 64 + c : c % H; };
+  auto there = [&](int c) { return row_of(c) < n_rows && head_of(c) < H && (H >= 64 || c < (64 / H) * H); };
+  const int c = ct * 16 + c16;
+  const bool col_ok = there(c);
+  const int col_pos = col_ok ? p_first + row_of(c) : -1;
+  const int col_lo = window > 0 ? col_pos - window + 1 : 0;
+  const int k_lo = window > 0 ? max(0, p_first - window + 1) : 0;     // the first key any column sees
+  const int s_first = k_lo / 32, s_end = p_last / 32 + 1;
+  const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
+  const long page_bytes = (long)PAGE * (KD + VD) * 2;
+
+  // the wave's copies: copy j = wave + 8 i brings 64 pieces of the buffer; a lane's piece by its page of the step (0, 1) and
+  // its bytes from the page's start
+  unsigned src_off[T8_LPW];
+  bool src_second[T8_LPW];
+#pragma unroll
+  for (int i = 0; i < T8_LPW; ++i) {
+    const int j = wave + 8 * i;
+    if (j < T8_KI) {
+      const int at = min(j * 64 + lane, 32 * T8_KPS - 1), key = at / T8_KPS, piece = min(at % T8_KPS, KD / 8 - 1);
+      src_second[i] = key >= PAGE;
+      src_off[i] = (unsigned)(((key & 15) * KD + piece * 8) * 2);
+    } else {
+      const int at = min((j - T8_KI) * 64 + lane, 4 * VD - 1), in_page = at % (2 * VD), ch = in_page >> 1;
+      src_second[i] = at >= 2 * VD;
+      src_off[i] = (unsigned)(PAGE * KD * 2 + ch * 32 + ((in_page & 1) ^ ((ch >> 3) & 1)) * 16);
+    }
+  }
+  auto stage = [&](int s, int buf) {
+    const int kb = s * 32;
+    const unsigned char* pg0 = (const unsigned char*)plane + (long)bt[kb >> 4] * page_bytes;
+    const unsigned char* pg1 = (const unsigned char*)plane + (long)bt[(kb >> 4) + (kb + 16 <= p_last ? 1 : 0)] * page_bytes;
+#pragma unroll
+    for (int i = 0; i < T8_LPW; ++i) {
+      const int j = wave + 8 * i;
+      if (j < T8_KI + T8_VI) lt_copy16((src_second[i] ? pg1 : pg0) + src_off[i], lds0 + buf * T8_STAGE + j * 1024);
+    }
+  };
+
+  bf16x8 qb[DC];
+#pragma unroll
+  for (int dc = 0; dc < DC; ++dc) {
+    const int d = dc * 32 + g * 8;
+    qb[dc] = (col_ok && d < KD) ? *reinterpret_cast<const bf16x8*>(q + (long)(row0 + row_of(c)) * ldq + (long)head_of(c) * KD + d) : zero8;
+  }
+  f32x4 o[T8_DB][4];
+#pragma unroll
+  for (int i = 0; i < T8_DB; ++i)
+#pragma unroll
+    for (int t = 0; t < 4; ++t) o[i][t] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+
+  stage(s_first, 0);
+  for (int s = s_first; s < s_end; ++s) {
+    const int kb = s * 32, buf = (s - s_first) & 1;
+    asm volatile("s_waitcnt vmcnt(0)" : : : "memory");                // this wave's pieces of the step are in LDS
+    __syncthreads();                                                  // ... and everyone's; everyone is done with the step before
+    if (s + 1 < s_end) stage(s + 1, buf ^ 1);
+    const unsigned char* st = lds + buf * T8_STAGE;
+    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int dc = 0; dc < DC; ++dc) {
+      const int d = dc * 32 + g * 8;
+      const bf16x8 k = d < KD ? *reinterpret_cast<const bf16x8*>(st + ((kt * 16 + c16) * T8_KPS + dc * 4 + g) * 16) : zero8;
+      if (dc & 1) s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, qb[dc], s1, 0, 0, 0);
+      else s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, qb[dc], s0, 0, 0, 0);
+    }
+    // the lane holds, for its column, the scores of the keys kb + 16 kt + 4g + i
+    const bool edge = kb + 31 > p_first || kb < (window > 0 ? p_last - window + 1 : 0);      // some column does not see all of the step
+    float sv[4], tmax = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      sv[i] = (s0[i] + s1[i]) * scale_log2;
+      if (edge) {
+        const int key = kb + kt * 16 + 4 * g + i;
+        sv[i] = (key <= col_pos && key >= col_lo) ? sv[i] : -INFINITY;
+      }
+      tmax = fmaxf(tmax, sv[i]);
+    }
+    tmax = quad_max(tmax);
+    if (g == 0) max_lds[kt * 64 + c] = tmax;
+    __syncthreads();
+    const float step_max = fmaxf(max_lds[c], max_lds[64 + c]);
+    const float m_new = step_max > m + 8.f ? step_max : m;            // (from -inf: the first step with a key)
+    const float m_use = m_new == -INFINITY ? 0.f : m_new;
+    const float alpha = m == m_new ? 1.f : exp2f(m - m_use);
+    bf16x4 p;
+    float psum = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float w = exp2f(sv[i] - m_use);
+      psum += w;
+      p[i] = static_cast<__bf16>(w);
+    }
+    *reinterpret_cast<bf16x4*>(p_lds + c * T8_P_STRIDE + (kt * 16 + 4 * g) * 2) = p;
+    if (kt == 0 && g == 0) alpha_lds[c] = alpha;
+    l = l * alpha + psum;
+    m = m_new;
+    __syncthreads();
+    // second product: lane (c16, g) brings the keys 8g .. 8g + 7 of the step for both operands
+    bf16x8 pb[4];
+    float al[4];
+    bool rescale = false;
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+      pb[t] = *reinterpret_cast<const bf16x8*>(p_lds + (t * 16 + c16) * T8_P_STRIDE + g * 16);
+      al[t] = alpha_lds[t * 16 + c16];
+      rescale |= al[t] != 1.f;
+    }
+    if (__any(rescale)) {
+#pragma unroll
+      for (int i = 0; i < T8_DB; ++i)
+#pragma unroll
+        for (int t = 0; t < 4; ++t)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) o[i][t][e] *= al[t];
+    }
+    const bool outside = kb + 31 > p_last || kb < k_lo;               // some of the step's slots hold nothing any column sees
+#pragma unroll
+    for (int i = 0; i < T8_DB; ++i) {
+      const int ch = min(wave + 8 * i, DB - 1) * 16 + c16;
+      bf16x8 va = *reinterpret_cast<const bf16x8*>(st + T8_V_AT + ((g >> 1) * 2 * VD + ch * 2 + ((g & 1) ^ ((ch >> 3) & 1))) * 16);
+      if (outside) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const int key = kb + 8 * g + e;
+          if (key > p_last || key < k_lo) va[e] = static_cast<__bf16>(0.f);
+        }
+      }
+#pragma unroll
+      for (int t = 0; t < 4; ++t) o[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va, pb[t], o[i][t], 0, 0, 0);
+    }
+  }
+  l = quad_sum(l);
+  __syncthreads();
+  if (g == 0) sum_lds[kt * 64 + c] = l;
+  if (kt == 0 && g == 0) max_lds[c] = m;
+  __syncthreads();
+  // the lane holds, for column t * 16 + c16, the channels db * 16 + 4g + e of its wave's blocks
+#pragma unroll
+  for (int t = 0; t < 4; ++t) {
+    const int cc = t * 16 + c16;
+    if (!there(cc)) continue;
+    const int head = head_of(cc);
+    const float inv = 1.f / (sum_lds[cc] + sum_lds[64 + cc] + sink_share(sinks, head, max_lds[cc]));
+    bf16* dst = out + (long)(row0 + row_of(cc)) * ldo + (long)head * VD + 4 * g;
+#pragma unroll
+    for (int i = 0; i < T8_DB; ++i) {
+      const int db = wave + 8 * i;
+      if (db >= DB) continue;
+      bf16x4 w;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) w[e] = static_cast<__bf16>(o[i][t][e] * inv);
+      *reinterpret_cast<bf16x4*>(dst + db * 16) = w;
+    }
+  }
+}
+
 // out[row, head, :] = sum_s 2^(m_s - M) o_s / sum_s 2^(m_s - M) l_s over a (row, head)'s splits, in a fixed order
 __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restrict__ part_o, const float2* __restrict__ part_ml,
                                                            bf16* __restrict__ out, long ldo, int H, int n_splits,
@@ -408,6 +612,12 @@ TIS_EXPORT int tis_attention_latent(const void* q, long ldq, const void* plane, 
   if (n_splits == 0) {
     if (!items) return tis_fail("attention_latent: the four-wave kernel needs its list of items");
     dim3 tgrid(n_items, (H + 63) / 64);
+    if (T8_FITS) {
+      latent_tile8_kernel<T8_FITS><<<tgrid, 512, 0, stream>>>((const bf16*)q, ldq, (const bf16*)plane, block_tables, bt_ld, row_seq,
+                                                             positions, (const int2*)items, (bf16*)out, ldo, H,
+                                                             scale * 1.4426950408889634f, window, sinks);
+      return tis_launch_status("attention_latent tiles");
+    }
     latent_tile_kernel<<<tgrid, 256, 0, stream>>>((const bf16*)q, ldq, (const bf16*)plane, block_tables, bt_ld, row_seq,
                                                   positions, (const int2*)items, (bf16*)out, ldo, H,
                                                   scale * 1.4426950408889634f, window, sinks);
