@@ -253,6 +253,22 @@ def test_a_product_per_head_with_a_gate(n, Hq, N, K, dtype):
     close(ops.rmsnorm32(z.cuda()[:, 5:5 + 2 * N], gain.cuda(), 1e-5), ref.rmsnorm32(z[:, 5:5 + 2 * N], gain, 1e-5), dtype, "norm of a part of a row")
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("M,N,K", [(1, 40, 64), (8, 96, 256), (8, 2304, 512), (33, 100, 40), (200, 128, 192), (700, 1028, 264), (300, 30, 64), (17, 24, 27)])
+def test_a_product_with_an_activation(M, N, K, dtype):
+    """Both few-row kernels, the tiled product, a width that only the few-row kernel takes at many rows, and rows that only the
+    plain product takes."""
+    ops, ref = hip_ops(dtype), TorchOps("cpu", DT[dtype])
+    g = torch.Generator().manual_seed(M + N)
+    x, w = (2 * torch.randn(M, K, generator=g)).to(DT[dtype]), (torch.randn(N, K, generator=g) / K ** 0.5).to(DT[dtype])
+    for act in ("gelu_tanh", "relu2", "silu"):
+        close(ops.linear_act(x.cuda(), w.cuda(), act), ref.linear_act(x, w, act), dtype, act)
+    big = (40 * torch.randn(M, K, generator=g)).to(DT[dtype])          # far into both tails
+    a = ops.linear_act(big.cuda(), w.cuda(), "gelu_tanh")
+    assert torch.isfinite(a.float()).all()
+    close(a, ref.linear_act(big, w, "gelu_tanh"), dtype, "tails")
+
+
 # ---- the engine ------------------------------------------------------------------------------------------------
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])

@@ -74,10 +74,14 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(
   const long page_stride = (long)PAGE * (KD + VD);
   const int last_page = pos / PAGE, first_page = k_lo / PAGE;
 
-  for (int i = tid; i < 16 * (KD / 8); i += 256) {
-    const int col = i / (KD / 8), piece = i % (KD / 8);
-    *reinterpret_cast<bf16x8*>(q_lds + col * DQ_STRIDE + piece * 8) =
-        hb * 16 + col < H ? *reinterpret_cast<const bf16x8*>(q + row * ldq + (long)(hb * 16 + col) * KD + piece * 8) : zero8;
+  // (the queries are asked for first and put into LDS once the first keys and values have been asked for, too)
+  constexpr int QN = (2 * KD + 255) / 256;
+  bf16x8 qreg[QN];
+#pragma unroll
+  for (int j = 0; j < QN; ++j) {
+    const int i = tid + j * 256, col = i / (KD / 8), piece = i % (KD / 8);
+    qreg[j] = (i < 2 * KD && hb * 16 + col < H)
+                  ? *reinterpret_cast<const bf16x8*>(q + row * ldq + (long)(hb * 16 + col) * KD + piece * 8) : zero8;
   }
   f32x4 o[DEC_DB];
 #pragma unroll
@@ -104,7 +108,14 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(
       for (int j = 0; j < DEC_PAGES; ++j)
         v[i][j] = *reinterpret_cast<const bf16x4*>(pg[j] + (long)PAGE * KD + (long)(db * 16 + c16) * PAGE + 4 * g);
     }
-    if (chunk == c_begin) __syncthreads();                          // the queries are there
+    if (chunk == c_begin) {
+#pragma unroll
+      for (int j = 0; j < QN; ++j) {
+        const int i = tid + j * 256, col = i / (KD / 8), piece = i % (KD / 8);
+        if (i < 2 * KD) *reinterpret_cast<bf16x8*>(q_lds + col * DQ_STRIDE + piece * 8) = qreg[j];
+      }
+      __syncthreads();
+    }
     f32x4 st0 = {0.f, 0.f, 0.f, 0.f}, st1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int dc = 0; dc < DC; ++dc) {
