@@ -148,8 +148,8 @@ def plain_logits(key, cfg, w64, ids):
 
 
 def errors(key, cfg, w64, reqs: Dict[str, List[int]], got) -> list:
-    """Sorted (error, place) over all places that came back: the difference of the logits with its mean taken off, root
-    mean square over the vocabulary, over the spread of the plain logits of that request."""
+    """Sorted (error, place) over all places that came back: the centred difference of the logits' root mean square, as a
+    share of the spread of that request's plain logits."""
     errs = []
     for rid, ids in reqs.items():
         want = plain_logits(key, cfg, w64, ids)

@@ -36,7 +36,7 @@ def read_streams(X, weights):
 
 
 def write_streams(X, mix, out, y):
-    """All streams at once from the old ones: X_t <- sum_s mix[s, t] X_s + out[t] y."""
+    """Every new stream from all the old ones: X_t <- sum_s mix[s, t] X_s + out[t] y."""
     return torch.einsum("st,slw->tlw", mix, X) + out.view(-1, 1, 1) * y
 
 

@@ -1,6 +1,6 @@
 // A residual of S streams in 32-bit: the end of one sublayer and the beginning of the next in one pass over a row.
 //
-//   X_t <- sum_s mix[s][t] X_s + out[t] (y + bias)     all streams at once from the old ones (y null: X stays as it is)
+//   X_t <- sum_s mix[s][t] X_s + out[t] (y + bias)     every new stream from all the old ones (y null: X stays as it is)
 //   u = sum_t read[t] X_t;  h = u / sqrt(mean(u^2) + eps) * gain
 //   h' = h + (h_before - h) * amount                   (amount null: h' = h), in the compute type
 //
